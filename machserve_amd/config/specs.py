@@ -49,9 +49,20 @@ class YarnSpec:
 
 
 @dataclass(frozen=True)
+class WavelengthScalingSpec:
+    """Scaling of a rotation's frequencies by their wavelength ``l = 2 pi / f`` (the scheme of Llama 3.1): a frequency whose
+    wavelength is below ``original / high`` stays, one above ``original / low`` becomes ``f / factor``, and in between, with
+    ``s = (original / l - low) / (high - low)``, it is ``(1 - s) f / factor + s f``.  Cosines and sines are not scaled."""
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass(frozen=True)
 class RotarySpec:
     """Rotation of pairs ``(j, j + rotary_dim/2)`` with ``freq_j = theta^(-2j/rotary_dim)``, or those frequencies
-    scaled as ``yarn`` says."""
+    scaled as ``yarn`` or ``wavelengths`` says."""
     kind: str
     head_dim: int
     theta: float
@@ -65,6 +76,7 @@ class RotarySpec:
     # which numbers of the rotated part make a pair: "halves" (j, j + rotary_dim/2) or "neighbours" (2j, 2j + 1); the
     # table of frequencies is the same, the pairing is the business of the mixer's kernel
     pairing: str = "halves"
+    wavelengths: Optional[WavelengthScalingSpec] = None
 
 
 @dataclass(frozen=True)
@@ -254,7 +266,10 @@ class ChunkedAttentionSpec:
     ``position``: the rotation of q and k (its ``rotary_dim`` first numbers of a head, pairs as its ``pairing`` says; None:
     none); ``score = scale q . k``, then with ``softcap`` ``softcap tanh(score / softcap)``; a row at position i sees the
     keys j <= i with ``floor(i / chunk) = floor(j / chunk)`` (``chunk`` None: every j <= i) and, with ``window``, ``i - j <
-    window``; softmax; output projection."""
+    window``; softmax; output projection.  With ``head_norm`` (in ``qk_norm``'s place) the RMS norm is over each head of q and
+    of k by itself, with one weight of ``head_dim`` for all query heads and one for all key heads.  ``sink``: the softmax's
+    denominator also holds ``exp(sink_h)``, a learned number per head without key or value.  ``head_gate``: head h's output is
+    multiplied by ``sigmoid(W_g x)_h`` ("g.weight", ``[heads, hidden]``)."""
     kind: str
     hidden: int
     heads: int
@@ -271,6 +286,9 @@ class ChunkedAttentionSpec:
     chunk: Optional[int] = None
     window: Optional[int] = None
     tensors: Mapping[str, str] = field(default_factory=dict)
+    head_norm: bool = False
+    sink: bool = False
+    head_gate: bool = False
 
 
 @dataclass(frozen=True)
@@ -335,10 +353,26 @@ class RoutedMlpSpec:
     # the router has this many outputs more, which stand for experts without tensors that return their input
     identity: int = 0
     # "softmax_chosen": the weights are the softmax over the chosen logits; "softmax_all": scores are the softmax over
-    # every router output, and the weights the chosen scores over their sum (+ 1e-20)
+    # every router output, and the weights the chosen scores over their sum (+ 1e-20); "sigmoid": the weights are the
+    # sigmoids of the chosen logits as they are
     scoring: str = "softmax_chosen"
     # with "softmax_all": a vector ("correction") added to the scores for the choice only
     correction: bool = False
+    # what a chosen expert's weight multiplies: its "output", or its "input" (gated experts: ``expert(w x)``)
+    weigh: str = "output"
+    # the expert that every token uses is multiplied by ``sigmoid(W_sg x)``, one number a token ("shared.gate_weight")
+    shared_gate: bool = False
+
+
+@dataclass(frozen=True)
+class PlainMlpSpec:
+    """``W_down act(W_up x)`` without a gate branch and without biases; ``activation``: "relu2" (the square of relu), "silu" or
+    "gelu_tanh"."""
+    kind: str
+    hidden: int
+    intermediate: int
+    activation: str = "relu2"
+    tensors: Mapping[str, str] = field(default_factory=dict)
 
 
 @dataclass(frozen=True)
@@ -386,6 +420,18 @@ class PostNormLayerSpec:
     feed_forward: Optional[object]
     mixer_post_norm: object
     feed_forward_post_norm: Optional[object]
+
+
+@dataclass(frozen=True)
+class SumNormLayerSpec:
+    """A block whose norms come after the sums: ``x <- norm(alpha x + mixer(x))``, then ``x <- norm(alpha x +
+    feed_forward(x))``; the branches read the stream itself.  ``feed_forward`` None: the layer has none."""
+    block: str
+    mixer: object
+    feed_forward: Optional[object]
+    mixer_norm: object
+    feed_forward_norm: Optional[object]
+    alpha: float = 1.0
 
 
 @dataclass(frozen=True)

@@ -158,6 +158,16 @@ __device__ __forceinline__ float gate_activation(float g, int act) {
 #endif
 }
 
+// ---- the activation of a feed-forward without a gate branch --------------------------
+enum UnaryActivation { UNARY_RELU2 = 0, UNARY_SILU = 1, UNARY_GELU_TANH = 2, UNARY_COUNT = 3 };
+__device__ __forceinline__ float unary_activation(float v, int act) {
+    if (act == UNARY_RELU2) {  // the square of relu
+        const float r = fmaxf(v, 0.f);
+        return r * r;
+    }
+    return gate_activation(v, act == UNARY_SILU ? ACT_SILU : ACT_GELU_TANH);
+}
+
 // ---- reductions -----------------------------------------------------------------
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -393,6 +393,199 @@ __global__ __launch_bounds__(256) void finish_rows_kernel(FinishArgs a) {
     }
 }
 
+// ---- rows of q, k, v and a gate per head from the partial sums of their product, q and k normed head by head ---------------
+// An RMS norm over each head of q and of k (one weight of d numbers for all query heads, one for all key heads; null: none),
+// then the rotation, the writes and the fillings of the kernel above; the gate's columns (behind v) go through a sigmoid
+// and are left as 32-bit factors, one per (row, head).
+struct HeadRowArgs {
+    const float* proj;      // [n_partials, T, stride]: q [H, d], k [KV, d], v [KV, dv], gate [H] (gate only if gate_out)
+    int n_partials;
+    size_t partial_stride;
+    int stride;
+    const float* q_norm;    // [d] or null
+    const float* k_norm;    // [d] or null
+    float eps;
+    const int* positions;   // [T]
+    const float* inv_freq;  // [rot / 2] or null: no rotation
+    int rot, neighbours;
+    const int* slot_map;    // [T] page * ps + offset
+    elem_t* q_out;          // [T, H * dp]
+    elem_t* kpool;          // [pages, KV, ps, dp]
+    elem_t* vpool;          // [pages, KV, dp, ps]
+    float* gate_out;        // [T, H] or null
+    int H, KV, d, dv, dp, ps;
+};
+
+// Any sizes: the row lies in LDS, a wave sums a head's squares.
+__global__ __launch_bounds__(256) void head_row_kernel(HeadRowArgs a) {
+    extern __shared__ float lds[];
+    const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, heads = a.H + a.KV, half = a.rot / 2;
+    const int nqk = heads * a.d, nv = a.KV * a.dv, n = nqk + nv + (a.gate_out ? a.H : 0);
+    float* row = lds;               // n floats
+    float* cs = row + n;            // half cosines, then half sines
+    float* inv = cs + a.rot;        // H + KV factors
+    for (int c = threadIdx.x; c < n; c += 256) {
+        float v = 0.f;
+#pragma unroll 8
+        for (int p = 0; p < a.n_partials; ++p) v += a.proj[p * a.partial_stride + (size_t)t * a.stride + c];
+        row[c] = v;
+    }
+    for (int j = threadIdx.x; j < half; j += 256) {
+        float c, s;
+        sincosf((float)a.positions[t] * a.inv_freq[j], &s, &c);
+        cs[j] = c;
+        cs[half + j] = s;
+    }
+    __syncthreads();
+    for (int h = wave; h < heads; h += 4) {
+        float ss = 0.f;
+        for (int e = lane; e < a.d; e += 64) ss += row[h * a.d + e] * row[h * a.d + e];
+        ss = wave_sum(ss);
+        if (lane == 0) inv[h] = (h < a.H ? a.q_norm : a.k_norm) ? 1.0f / sqrtf(ss / (float)a.d + a.eps) : 1.0f;
+    }
+    __syncthreads();
+    const int slot = a.slot_map[t];
+    const int page = slot >= 0 ? slot / a.ps : 0, off = slot >= 0 ? slot % a.ps : 0;
+    for (int c = threadIdx.x; c < nqk; c += 256) {
+        const int h = c / a.d, i = c - h * a.d;
+        const bool is_q = h < a.H;
+        const float* nw = is_q ? a.q_norm : a.k_norm;
+        const float* base = row + h * a.d;
+        auto normed = [&](int e) { return base[e] * inv[h] * (nw ? nw[e] : 1.0f); };
+        float v;
+        if (i >= a.rot) {
+            v = normed(i);
+        } else if (a.neighbours) {
+            const int pr = i >> 1;
+            v = (i & 1) ? normed(i) * cs[pr] + normed(i - 1) * cs[half + pr] : normed(i) * cs[pr] - normed(i + 1) * cs[half + pr];
+        } else {
+            v = i < half ? normed(i) * cs[i] - normed(i + half) * cs[half + i] : normed(i) * cs[i - half] + normed(i - half) * cs[i];
+        }
+        if (is_q) a.q_out[((size_t)t * a.H + h) * a.dp + i] = from_f32<elem_t>(v);
+        else if (slot >= 0) a.kpool[(((size_t)page * a.KV + h - a.H) * a.ps + off) * a.dp + i] = from_f32<elem_t>(v);
+    }
+    const int fill = a.dp - a.d;
+    for (int c = threadIdx.x; c < a.H * fill; c += 256)
+        a.q_out[((size_t)t * a.H + c / fill) * a.dp + a.d + c % fill] = from_f32<elem_t>(0.f);
+    if (slot >= 0)
+        for (int c = threadIdx.x; c < nv; c += 256) {
+            const int h = c / a.dv, e = c - h * a.dv;
+            a.vpool[(((size_t)page * a.KV + h) * a.dp + e) * a.ps + off] = from_f32<elem_t>(row[nqk + c]);
+        }
+    if (a.gate_out)
+        for (int h = threadIdx.x; h < a.H; h += 256) a.gate_out[(size_t)t * a.H + h] = 1.0f / (1.0f + expf(-row[nqk + nv + h]));
+}
+
+// The same without a row in LDS, for heads and rotated parts that are multiples of 8, values that are a multiple of 4 and
+// up to NP partial sums.  L lanes (a power of two, at least d / 8) hold a head, eight numbers each as two quads: lanes of the
+// rotated part both quads of four pairs (j, j + rot / 2), or four pairs of neighbours; the others eight numbers that pass.
+// All of a quad's sums are asked for before the first is used, a head's squares are summed over its lanes by shuffles.
+// The items are laid out so that a head never straddles a wave and a wave holds one kind of item.
+template <int NP>
+__global__ __launch_bounds__(256) void head_row_quads_kernel(HeadRowArgs a, int L) {
+    __shared__ float cs[256], sn[256];
+    const int t = blockIdx.x, half = a.rot / 2;
+    const int slot = a.slot_map[t];
+    for (int j = threadIdx.x; j < half; j += 256) {
+        float c, s;
+        sincosf((float)a.positions[t] * a.inv_freq[j], &s, &c);
+        cs[j] = c;
+        sn[j] = s;
+    }
+    __syncthreads();
+    const int page = slot >= 0 ? slot / a.ps : 0, off = slot >= 0 ? slot % a.ps : 0;
+    const float* rowp = a.proj + (size_t)t * a.stride;
+    auto summed = [&](int c) {  // the partial sums of columns c .. c + 3, in order
+        f32x4 v[NP];
+#pragma unroll
+        for (int p = 0; p < NP; ++p) v[p] = *reinterpret_cast<const f32x4*>(rowp + (size_t)min(p, a.n_partials - 1) * a.partial_stride + c);
+        f32x4 r = v[0];
+#pragma unroll
+        for (int p = 1; p < NP; ++p) r += v[p] * (p < a.n_partials ? 1.f : 0.f);
+        return r;
+    };
+    auto store_quad = [](elem_t* o, const f32x4& v) {
+#ifdef MS_ELEM_HALF
+        half4_t b = {(elem_t)v[0], (elem_t)v[1], (elem_t)v[2], (elem_t)v[3]};
+        *reinterpret_cast<half4_t*>(o) = b;
+#else
+        *reinterpret_cast<f32x4*>(o) = v;
+#endif
+    };
+    const int heads = a.H + a.KV, nqk = heads * a.d, nv = a.KV * a.dv;
+    const int per = a.d / 8, rot_lanes = a.rot / 8;
+    const int n_head = ceil_div(heads * L, 64) * 64;              // items of q and k heads, whole waves
+    const int n_vq = nv / 4, n_v = ceil_div(n_vq, 64) * 64;      // quads of values, whole waves
+    const int n_items = n_head + n_v + (a.gate_out ? a.H : 0);
+    for (int it = threadIdx.x; it < n_items; it += 256) {  // (256 is whole waves: what follows is the same branch for a wave)
+        if (it < n_head) {
+            const int h_raw = it / L, l_raw = it % L;
+            const bool live = h_raw < heads && l_raw < per;
+            const int h = min(h_raw, heads - 1), l = min(l_raw, per - 1);
+            int j0, j1;
+            if (l < rot_lanes && !a.neighbours) { j0 = 4 * l; j1 = half + 4 * l; }
+            else { j0 = 8 * l; j1 = j0 + 4; }
+            const float* nw = h < a.H ? a.q_norm : a.k_norm;
+            f32x4 x0 = summed(h * a.d + j0), x1 = summed(h * a.d + j1);
+            f32x4 w0 = (f32x4){1.f, 1.f, 1.f, 1.f}, w1 = w0;
+            if (nw) {
+                w0 = *reinterpret_cast<const f32x4*>(nw + j0);
+                w1 = *reinterpret_cast<const f32x4*>(nw + j1);
+            }
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss += x0[e] * x0[e] + x1[e] * x1[e];
+            ss = live ? ss : 0.f;
+            for (int o = L / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+            const float inv = nw ? 1.0f / sqrtf(ss / (float)a.d + a.eps) : 1.0f;
+            x0 = x0 * inv * w0;
+            x1 = x1 * inv * w1;
+            f32x4 y0 = x0, y1 = x1;
+            if (l < rot_lanes) {
+                if (a.neighbours) {
+#pragma unroll
+                    for (int e = 0; e < 4; e += 2) {
+                        const int p0 = 4 * l + e / 2, p1 = p0 + 2;
+                        y0[e] = x0[e] * cs[p0] - x0[e + 1] * sn[p0];
+                        y0[e + 1] = x0[e + 1] * cs[p0] + x0[e] * sn[p0];
+                        y1[e] = x1[e] * cs[p1] - x1[e + 1] * sn[p1];
+                        y1[e + 1] = x1[e + 1] * cs[p1] + x1[e] * sn[p1];
+                    }
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        y0[e] = x0[e] * cs[j0 + e] - x1[e] * sn[j0 + e];
+                        y1[e] = x1[e] * cs[j0 + e] + x0[e] * sn[j0 + e];
+                    }
+                }
+            }
+            if (!live) continue;
+            elem_t* o;
+            if (h < a.H) o = a.q_out + ((size_t)t * a.H + h) * a.dp;
+            else if (slot >= 0) o = a.kpool + (((size_t)page * a.KV + (h - a.H)) * a.ps + off) * a.dp;
+            else continue;
+            store_quad(o + j0, y0);
+            store_quad(o + j1, y1);
+            if (h < a.H && l == 0)
+                for (int e = a.d; e < a.dp; e += 4) store_quad(o + e, (f32x4){0.f, 0.f, 0.f, 0.f});
+        } else if (it < n_head + n_v) {
+            const int q = it - n_head;
+            if (q >= n_vq || slot < 0) continue;
+            const int per_v = a.dv / 4, h = q / per_v, dd = (q % per_v) * 4;
+            const f32x4 v = summed(nqk + h * a.dv + dd);
+            elem_t* o = a.vpool + (((size_t)page * a.KV + h) * a.dp + dd) * a.ps + off;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[(size_t)e * a.ps] = from_f32<elem_t>(v[e]);
+        } else {
+            const int h = it - n_head - n_v;
+            float v = 0.f;
+#pragma unroll
+            for (int p = 0; p < NP; ++p) v += p < a.n_partials ? rowp[(size_t)p * a.partial_stride + nqk + nv + h] : 0.f;
+            a.gate_out[(size_t)t * a.H + h] = 1.0f / (1.0f + expf(-v));
+        }
+    }
+}
+
 // Differential attention behind the attention kernel.  o [T, 2 H maps, dp]: the maps of a key/value head's group lie side
 // by side, (key/value head, map, head of the group).  A head's result is map 0 minus lam times map 1 over its first dv
 // numbers, divided by its root mean square, times `factor`, times sigmoid(gate); heads side by side in rows of ld_out
@@ -472,6 +665,32 @@ extern "C" int ms_finish_rows(const float* rows, int stride, const float* q_norm
                  (elem_t*)vpool, H, KV, d, dv, dp, ps};
     hipLaunchKernelGGL(finish_rows_kernel, dim3(T), dim3(256), (size_t)(stride + rot) * sizeof(float), stream, a);
     return check_launch("finish_rows");
+}
+
+// proj float [n_partials, T, stride]; norms of d numbers or null; gate_out null or float [T, H].
+extern "C" int ms_finish_heads(const float* proj, int n_partials, int stride, const float* q_norm, const float* k_norm, float eps,
+                               const int* positions, const float* inv_freq, int rot, int neighbours, const int* slot_map, void* q_out,
+                               void* kpool, void* vpool, float* gate_out, int T, int H, int KV, int d, int dv, int dp, int ps, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && n_partials >= 1 && H > 0 && KV > 0 && d > 0 && dv > 0 && dp >= d && dp >= dv && ps > 0,
+               "finish heads: %d rows, %d partial sums, %d / %d heads of %d and %d in %d", T, n_partials, H, KV, d, dv, dp);
+    const int n = (H + KV) * d + KV * dv + (gate_out ? H : 0);
+    if (!inv_freq) rot = 0;
+    MS_REQUIRE(stride >= n && n + rot + H + KV <= CONV_MAX_ROW, "finish heads: a row of %d numbers (stride %d, at most %d)", n, stride, CONV_MAX_ROW);
+    MS_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= d, "finish heads: %d of %d numbers of a head are rotated", rot, d);
+    HeadRowArgs a{proj, n_partials, (size_t)T * stride, stride, q_norm, k_norm, eps, positions, inv_freq, rot, neighbours, slot_map,
+                  (elem_t*)q_out, (elem_t*)kpool, (elem_t*)vpool, gate_out, H, KV, d, dv, dp, ps};
+    const bool aligned = ((reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(q_norm) | reinterpret_cast<uintptr_t>(k_norm) |
+                           reinterpret_cast<uintptr_t>(q_out) | reinterpret_cast<uintptr_t>(kpool)) & 15) == 0;
+    if (aligned && d % 8 == 0 && d <= 512 && rot % 8 == 0 && rot <= 512 && dv % 4 == 0 && dp % 4 == 0 && stride % 4 == 0 && n_partials <= 8) {
+        int L = 1;
+        while (L < d / 8) L *= 2;
+        if (n_partials == 1) hipLaunchKernelGGL(head_row_quads_kernel<1>, dim3(T), dim3(256), 0, stream, a, L);
+        else if (n_partials <= 4) hipLaunchKernelGGL(head_row_quads_kernel<4>, dim3(T), dim3(256), 0, stream, a, L);
+        else hipLaunchKernelGGL(head_row_quads_kernel<8>, dim3(T), dim3(256), 0, stream, a, L);
+    } else {
+        hipLaunchKernelGGL(head_row_kernel, dim3(T), dim3(256), (size_t)(n + rot + H + KV) * sizeof(float), stream, a);
+    }
+    return check_launch("finish_heads");
 }
 
 extern "C" int ms_diff_combine(const void* o, const float* gate, void* out, float lam, float eps, float factor, int T, int H, int KV, int dp,

@@ -234,6 +234,86 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, co
     for (int c = threadIdx.x; c < d; c += 256) dst[c] += vals[c] * inv * w[c];
 }
 
+// x[t, :] = v / sqrt(mean(v^2) + eps) * w with v = alpha * x[t, :] + sum_p partials[p, t, :] (in order) + bias: the norm that
+// comes after a residual sum.  The row also goes out in the element type (`out`, null where that is float: x itself is the
+// row then), which is what the next branch reads.  This form takes any width and any number of sums.
+__global__ __launch_bounds__(256) void sum_norm_kernel(float* __restrict__ x, const float* __restrict__ partials, int n_partials,
+                                                       size_t partial_stride, const float* __restrict__ bias, float alpha,
+                                                       const float* __restrict__ w, elem_t* __restrict__ out, int d, float eps) {
+    __shared__ float scratch[4];
+    extern __shared__ float vals[];  // d floats: the summed row
+    const size_t r = blockIdx.x;
+    float* row = x + r * d;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < d; c += 256) {
+        float y = 0.f;
+#pragma unroll 8
+        for (int p = 0; p < n_partials; ++p) y += partials[(size_t)p * partial_stride + r * d + c];
+        const float v = alpha * row[c] + (y + (bias ? bias[c] : 0.f));
+        vals[c] = v;
+        ss += v * v;
+    }
+    ss = block_sum<256>(ss, scratch);
+    const float inv = 1.0f / sqrtf(ss / (float)d + eps);
+    for (int c = threadIdx.x; c < d; c += 256) {  // a thread meets its own columns again
+        const float v = vals[c] * inv * w[c];
+        row[c] = v;
+        if (out) out[r * d + c] = from_f32<elem_t>(v);
+    }
+}
+
+// The same for widths that are a multiple of four and at most 1024 * G, and up to NP sums: a thread owns G groups of four
+// columns and asks for everything the row needs before it uses the first value (sums beyond the last one read the last one
+// again and count for nothing).
+template <int G, int NP>
+__global__ __launch_bounds__(256) void sum_norm_wide_kernel(float* __restrict__ x, const float* __restrict__ partials, int n_partials,
+                                                            size_t partial_stride, const float* __restrict__ bias, float alpha,
+                                                            const float* __restrict__ w, elem_t* __restrict__ out, int d, float eps) {
+    arguments_now(x, partials, n_partials, partial_stride, bias, alpha, w, out, d, eps);
+    __shared__ float scratch[4];
+    const size_t r = blockIdx.x;
+    const int ng = d / 4;
+    f32x4* row = reinterpret_cast<f32x4*>(x + r * d);
+    const f32x4* src = reinterpret_cast<const f32x4*>(partials + r * d);
+    const size_t stride4 = partial_stride / 4;
+    f32x4 v[G], wv[G], bv[G], q[NP][G];
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        const int c4 = threadIdx.x + g * 256, at = c4 < ng ? c4 : 0;  // a group beyond the row reads group 0 and is dropped
+        v[g] = row[at];
+        wv[g] = reinterpret_cast<const f32x4*>(w)[at];
+        bv[g] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int p = 0; p < NP; ++p) q[p][g] = src[(size_t)min(p, n_partials - 1) * stride4 + at];
+    }
+    if (bias)
+#pragma unroll
+        for (int g = 0; g < G; ++g) {
+            const int c4 = threadIdx.x + g * 256;
+            bv[g] = reinterpret_cast<const f32x4*>(bias)[c4 < ng ? c4 : 0];
+        }
+    float ss = 0.f;
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        f32x4 y = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int p = 0; p < NP; ++p) y += q[p][g] * (p < n_partials ? 1.f : 0.f);
+        v[g] = v[g] * alpha + (y + bv[g]);
+        if (threadIdx.x + g * 256 < ng) ss += v[g].x * v[g].x + v[g].y * v[g].y + v[g].z * v[g].z + v[g].w * v[g].w;
+    }
+    ss = block_sum<256>(ss, scratch);
+    const float inv = 1.0f / sqrtf(ss / (float)d + eps);
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        const int c4 = threadIdx.x + g * 256;
+        if (c4 >= ng) continue;
+        const f32x4 o = v[g] * inv * wv[g];
+        row[c4] = o;
+        typedef elem_t out4_t __attribute__((ext_vector_type(4)));
+        if (out) *reinterpret_cast<out4_t*>(out + r * d + (size_t)c4 * 4) = (out4_t){from_f32<elem_t>(o.x), from_f32<elem_t>(o.y), from_f32<elem_t>(o.z), from_f32<elem_t>(o.w)};
+    }
+}
+
 // Two branches side by side, each given as the partial sums of its last product: every branch's sum is normalised with
 // a weight of its own, half their sum is normalised again, and that is added to the stream:
 // y = (rms(a) * wa + rms(b) * wb) / 2;  x[t, :] += rms(y) * w.
@@ -599,6 +679,38 @@ extern "C" int ms_norm_add_bias(float* x, const float* partials, int n_partials,
     hipLaunchKernelGGL(norm_add_kernel, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, (size_t)T * d, w,
                        d, eps, bias);
     return check_launch("norm_add");
+}
+
+// x [T, d] <- rmsnorm(alpha x + sum of partials [n_partials, T, d] + bias) * w; out [T, d] in the element type, or null.
+extern "C" int ms_sum_norm(float* x, const float* partials, int n_partials, const float* bias, float alpha, const float* w, void* out,
+                           int T, int d, float eps, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && d > 0 && n_partials > 0, "sum_norm: empty problem T=%d d=%d with %d sums", T, d, n_partials);
+    MS_REQUIRE(d <= MAX_ROW_FLOATS, "sum_norm: width %d exceeds the row buffer of %d", d, MAX_ROW_FLOATS);
+    MS_REQUIRE(x && partials && w, "sum_norm: a buffer is missing");
+    const size_t ps = (size_t)T * d;
+    const int groups = d % 4 == 0 ? (d <= 1024 ? 1 : (d <= 2048 ? 2 : (d <= 4096 ? 4 : 0))) : 0;
+    const bool aligned = (reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(partials) |
+                          reinterpret_cast<uintptr_t>(bias) | reinterpret_cast<uintptr_t>(out)) % 16 == 0;
+    if (groups && aligned && n_partials <= (groups == 4 ? 8 : 16)) {
+#define MS_SUM_NORM(G_, NP_)                                                                                                           \
+    hipLaunchKernelGGL((sum_norm_wide_kernel<G_, NP_>), dim3(T), dim3(256), 0, stream, x, partials, n_partials, ps, bias, alpha, w, \
+                       (elem_t*)out, d, eps)
+#define MS_SUM_NORM_NP(G_, MOST_)                        \
+    if (n_partials == 1) MS_SUM_NORM(G_, 1);             \
+    else if (n_partials == 2) MS_SUM_NORM(G_, 2);        \
+    else if (n_partials <= 4) MS_SUM_NORM(G_, 4);        \
+    else if (n_partials <= 8) MS_SUM_NORM(G_, 8);        \
+    else MS_SUM_NORM(G_, MOST_)
+        if (groups == 1) { MS_SUM_NORM_NP(1, 16); }
+        else if (groups == 2) { MS_SUM_NORM_NP(2, 16); }
+        else { MS_SUM_NORM_NP(4, 8); }
+#undef MS_SUM_NORM_NP
+#undef MS_SUM_NORM
+    } else {
+        hipLaunchKernelGGL(sum_norm_kernel, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, ps, bias, alpha, w,
+                           (elem_t*)out, d, eps);
+    }
+    return check_launch("sum_norm");
 }
 
 extern "C" int ms_pair_norm_add(float* x, const float* pa, int na, const float* wa, const float* pb, int nb, const float* wb,

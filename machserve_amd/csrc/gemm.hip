@@ -30,7 +30,7 @@ constexpr int EPC = 4;
 constexpr int KPAD = 8;  // rows of 160 bytes (BK 32)
 #endif
 
-enum EpiKind { EPI_STORE_F32 = 0, EPI_STORE_ELEM = 1, EPI_RESIDUAL = 2, EPI_SWIGLU = 3, EPI_QKV_ROPE = 4 };
+enum EpiKind { EPI_STORE_F32 = 0, EPI_STORE_ELEM = 1, EPI_RESIDUAL = 2, EPI_SWIGLU = 3, EPI_QKV_ROPE = 4, EPI_ACT = 5 };
 
 struct EpiArgs {
     void* out;          // [M, ldo]
@@ -44,7 +44,7 @@ struct EpiArgs {
     const float* row_ss;  // [ss_parts, M] or null
     int ss_parts;
     float ss_eps;
-    int act;            // SWIGLU: the activation on the gate (GateActivation)
+    int act;            // SWIGLU: the activation on the gate (GateActivation); ACT: the activation (UnaryActivation)
     // QKV_ROPE: the columns are H query heads, KV key heads and KV value heads of the tile's width; bias added, queries
     // and keys rotated by the rows' angles (pairs (j, j + half a head)), queries to `out` [M, H * hd], keys and values
     // into their pages
@@ -400,6 +400,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_kernel(const elem_t* __rest
                         const float v = acc[i][j][e] + b;
                         if constexpr (EPI == EPI_STORE_F32) reinterpret_cast<float*>(ep.out)[split * ep.split_stride + o] = v;
                         else if constexpr (EPI == EPI_STORE_ELEM) reinterpret_cast<elem_t*>(ep.out)[o] = from_f32<elem_t>(v);
+                        else if constexpr (EPI == EPI_ACT) reinterpret_cast<elem_t*>(ep.out)[o] = from_f32<elem_t>(unary_activation(v, ep.act));
                         else reinterpret_cast<float*>(ep.out)[o] += v;  // residual stream, 32-bit
                     }
                 }
@@ -600,6 +601,13 @@ extern "C" int ms_linear_swiglu(const void* a, const void* w, void* out, int M, 
     const int n = 2 * ceil_div(I, 16) * 16;
     EpiArgs ep{out, nullptr, I, I, 0, 0, nullptr, 0, 0.f, act};
     return launch_gemm<EPI_SWIGLU>((const elem_t*)a, (const elem_t*)w, M, n, K, ep, stream);
+}
+
+// out[M, N] = act(a[M, K] w[N, K]^T) in the element type, the activation (UnaryActivation) in the product's epilogue.
+extern "C" int ms_linear_act(const void* a, const void* w, void* out, int M, int N, int K, int act, hipStream_t stream) {
+    MS_REQUIRE(act >= 0 && act < UNARY_COUNT, "product with an activation: no activation %d", act);
+    EpiArgs ep{out, nullptr, N, N, 0, 0, nullptr, 0, 0.f, act};
+    return launch_gemm<EPI_ACT>((const elem_t*)a, (const elem_t*)w, M, N, K, ep, stream);
 }
 
 // Whether ms_linear_swiglu_scaled takes this shape: bfloat16, one tile of rows, whole K steps of 64.

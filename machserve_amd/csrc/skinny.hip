@@ -21,12 +21,12 @@ namespace ms {
 constexpr int KSTEP = 128;  // K elements per wave iteration: four fragments per lane; fragment c of the wave is the
                             // contiguous chunk c of 32 elements (the four key groups side by side: 64 bytes a row in bf16)
 
-enum SkinnyEpi { SK_STORE_F32 = 0, SK_SWIGLU = 1, SK_RESIDUAL = 2, SK_RESIDUAL_PRENORM = 3 };
+enum SkinnyEpi { SK_STORE_F32 = 0, SK_SWIGLU = 1, SK_RESIDUAL = 2, SK_RESIDUAL_PRENORM = 3, SK_ACT = 4 };
 
 struct SkinnyArgs {
     const elem_t* A;  // [M, K]
     const elem_t* W;  // [N, K]
-    void* out;        // SK_STORE_F32: float [gridDim.y, M, N]; SK_SWIGLU: elem [M, n_out]; SK_RESIDUAL: float [M, N], added to
+    void* out;        // SK_STORE_F32: float [gridDim.y, M, N]; SK_SWIGLU: elem [M, n_out]; SK_RESIDUAL: float [M, N], added to; SK_ACT: elem [M, N]
     int M, N, K;
     int k_per_wave;   // multiple of 32
     int n_out;        // SK_SWIGLU: intermediate size
@@ -39,7 +39,7 @@ struct SkinnyArgs {
     const float* row_ss;  // [ss_parts, M] or null
     int ss_parts;
     float ss_eps;
-    int act;          // SK_SWIGLU: the activation on the gate (GateActivation)
+    int act;          // SK_SWIGLU: the activation on the gate (GateActivation); SK_ACT: the activation (UnaryActivation)
 };
 
 // A block of eight waves puts two on every SIMD; with more than 128 registers a wave a CU then holds one
@@ -47,7 +47,7 @@ struct SkinnyArgs {
 // although every block only waits for its one trip to memory.  One row tile under at most 32 columns a wave
 // fits 128 registers where nothing of the residual stream is held beside the sums: two blocks a CU.
 template <int MT, int NT, int WN, int KSI, int EPI>
-constexpr int skinny_waves_per_simd() { return (WN * KSI == 8 && MT == 1 && NT <= 2 && EPI <= SK_SWIGLU) ? 4 : 1; }
+constexpr int skinny_waves_per_simd() { return (WN * KSI == 8 && MT == 1 && NT <= 2 && (EPI <= SK_SWIGLU || EPI == SK_ACT)) ? 4 : 1; }
 
 template <int MT, int NT, int WN, int KSI, int EPI>
 __global__ __launch_bounds__(64 * WN * KSI, (skinny_waves_per_simd<MT, NT, WN, KSI, EPI>())) void gemm_skinny_kernel(SkinnyArgs a) {
@@ -280,6 +280,20 @@ __global__ __launch_bounds__(64 * WN * KSI, (skinny_waves_per_simd<MT, NT, WN, K
                 if (r16 == 0 && row < a.M) a.ss_part[(size_t)(blockIdx.x * WN + wn) * a.M + row] = sq;
             }
         }
+    } else if constexpr (EPI == SK_ACT) {  // all of K lies in this block
+        if (!owner) return;
+        elem_t* out = reinterpret_cast<elem_t*>(a.out);
+#pragma unroll
+        for (int i = 0; i < MT; ++i)
+#pragma unroll
+            for (int j = 0; j < NT; ++j) {
+                const int col = n0 + j * 16 + r16;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int row = i * 16 + grp * 4 + e;
+                    if (row < a.M && col < a.N) out[(size_t)row * a.N + col] = from_f32<elem_t>(unary_activation(acc[i][j][e], a.act));
+                }
+            }
     } else {
         if (owner) {
             // SK_RESIDUAL: all of K lies in this block (gridDim.y == 1), so every element has one writer
@@ -602,6 +616,13 @@ extern "C" int ms_linear_swiglu_skinny(const void* a, const void* w, void* out, 
     const int n = 2 * ceil_div(I, 16) * 16;
     SkinnyArgs args{(const elem_t*)a, (const elem_t*)w, out, M, n, K, 0, I, nullptr, nullptr, nullptr, nullptr, 0, 0.f, act};
     return launch_skinny<SK_SWIGLU>(args, plan_skinny(M, n, K, false, true), stream);
+}
+
+// out[M, N] = act(a w^T) in the element type, the activation (UnaryActivation) in the epilogue.
+extern "C" int ms_linear_act_skinny(const void* a, const void* w, void* out, int M, int N, int K, int act, hipStream_t stream) {
+    MS_REQUIRE(act >= 0 && act < UNARY_COUNT, "product with an activation: no activation %d", act);
+    SkinnyArgs args{(const elem_t*)a, (const elem_t*)w, out, M, N, K, 0, 0, nullptr, nullptr, nullptr, nullptr, 0, 0.f, act};
+    return launch_skinny<SK_ACT>(args, plan_skinny(M, N, K, false), stream);
 }
 
 // Whether ms_linear_swiglu_scaled_skinny takes this shape, and is the faster of the two forms for it: one

@@ -384,6 +384,17 @@ class HipOps:
                                    _c_int(act), self._stream()))
         return out
 
+    def linear_act(self, a: torch.Tensor, w: torch.Tensor, activation: str) -> torch.Tensor:
+        """``act(a @ w.T)`` in the element type, the activation (one of :data:`UNARY_ACTIVATIONS`) in the product's epilogue."""
+        if activation not in UNARY_ACTIVATIONS:
+            raise KernelError(f"linear_act: activation {activation!r} is not built (built: {', '.join(sorted(UNARY_ACTIVATIONS))})")
+        M, N, K = self._mm_operands(a, w, "linear_act")
+        out = torch.empty((M, N), dtype=self.dtype, device=a.device)
+        fn = self._core.ms_linear_act if self._tiled(M, N, K) else self._core.ms_linear_act_skinny
+        self._check(self._core, fn(_ptr(a), _ptr(w), _ptr(out), _c_int(M), _c_int(N), _c_int(K), _c_int(UNARY_ACTIVATIONS[activation]),
+                                   self._stream()))
+        return out
+
     # ------------------------------------------------------------------ products with the norm folded in
     def norm_folds_into(self, M: int, N: int, K: int, n_partials: int) -> bool:
         """Whether a few-rows product over the stream can apply the stream's RMS norm itself (at most
@@ -988,6 +999,21 @@ class HipOps:
         self._check(self._core, self._core.ms_norm_add_bias(_ptr(x), _ptr(partials), _c_int(partials.shape[0]), _ptr(bias), _ptr(weight),
                                                             _c_int(T), _c_int(d), _c_float(eps), self._stream()))
 
+    def sum_norm(self, x: torch.Tensor, partials: torch.Tensor, bias: Optional[torch.Tensor], alpha: float, weight: torch.Tensor,
+                 eps: float) -> torch.Tensor:
+        """In place ``x = rmsnorm(alpha x + sum(partials) + bias) * weight``; returns the rows in the element type (``x`` itself
+        in the 32-bit build): the norm behind a residual sum, ``partials [P, T, d]`` being what a branch's last product left."""
+        T, d = x.shape
+        self._want(x, torch.float32, "sum_norm stream")
+        self._want(partials, torch.float32, "sum_norm sums", partials.shape[0], T, d)
+        if bias is not None:
+            self._want(bias, torch.float32, "sum_norm bias", d)
+        self._want(weight, torch.float32, "sum_norm weight", d)
+        out = None if self.dtype == torch.float32 else torch.empty((T, d), dtype=self.dtype, device=x.device)
+        self._check(self._core, self._core.ms_sum_norm(_ptr(x), _ptr(partials), _c_int(partials.shape[0]), _ptr(bias), _c_float(alpha),
+                                                       _ptr(weight), _ptr(out), _c_int(T), _c_int(d), _c_float(eps), self._stream()))
+        return x if out is None else out
+
     def pair_norm_add(self, x: torch.Tensor, pa: torch.Tensor, wa: torch.Tensor, pb: torch.Tensor, wb: torch.Tensor, weight: torch.Tensor,
                       eps: float) -> None:
         """``y = (rmsnorm(sum(pa)) * wa + rmsnorm(sum(pb)) * wb) / 2;  x += rmsnorm(y) * weight``: two branches side by side,
@@ -1071,6 +1097,39 @@ class HipOps:
                                             _ptr(vpool), _c_int(T), _c_int(H), _c_int(0 if queries_only else KV), _c_int(d), _c_int(dv), _c_int(dp),
                                             _c_int(page_size), self._stream()))
         return q
+
+    def finish_heads(self, proj: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], eps: float,
+                     positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rot: int, neighbours: bool, gated: bool,
+                     slot_map: torch.Tensor, kpool: torch.Tensor, vpool: torch.Tensor, H: int, KV: int, d: int, dv: int, page_size: int):
+        """Rows of a projection given as float32 partial sums ``[P, T, stride]`` (q ``[H, d]``, k ``[KV, d]``, v ``[KV, dv]``, then
+        with ``gated`` one gate column per head): an RMS norm over each head of q and of k (weights of ``d`` numbers; None:
+        none), the rotation of the first ``rot`` numbers of every head as in :meth:`finish_rows`, k and v written into their
+        pages.  Returns ``(q [T, H * dp]`` in the element type with ``dp`` the pools' head size, ``sigmoid(gate)`` float32 ``[T, H]`` or
+        None)``."""
+        lib = self._extra_lib("convattn")
+        if proj.dim() == 2:
+            proj = proj.unsqueeze(0)
+        P, T, stride = proj.shape
+        self._want(proj, torch.float32, "finish heads")
+        for w in (q_norm, k_norm):
+            if w is not None:
+                self._want(w, torch.float32, "head norm weight", d)
+        self._want(positions, torch.int32, "finish heads positions", T)
+        if inv_freq is not None:
+            self._want(inv_freq, torch.float32, "rotation frequencies", rot // 2)
+        else:
+            rot = 0
+        self._want(slot_map, torch.int32, "finish heads slot_map", T)
+        pages, _, _, dp = kpool.shape
+        self._want(kpool, self.dtype, "key pool", pages, KV, page_size, dp)
+        self._want(vpool, self.dtype, "value pool", pages, KV, dp, page_size)
+        q = torch.empty((T, H * dp), dtype=self.dtype, device=proj.device)
+        gate = torch.empty((T, H), dtype=torch.float32, device=proj.device) if gated else None
+        self._check(lib, lib.ms_finish_heads(_ptr(proj), _c_int(P), _c_int(stride), _ptr(q_norm), _ptr(k_norm), _c_float(eps), _ptr(positions),
+                                             _ptr(inv_freq), _c_int(rot), _c_int(int(neighbours)), _ptr(slot_map), _ptr(q), _ptr(kpool),
+                                             _ptr(vpool), _ptr(gate), _c_int(T), _c_int(H), _c_int(KV), _c_int(d), _c_int(dv), _c_int(dp),
+                                             _c_int(page_size), self._stream()))
+        return q, gate
 
     def diff_combine(self, o: torch.Tensor, gate: torch.Tensor, lam: float, eps: float, factor: float, H: int, KV: int, hd: int, dv: int,
                      out_cols: int) -> torch.Tensor:
@@ -1236,31 +1295,34 @@ class HipOps:
         return {"experts": self._extra_lib("routed").ms_route_max_experts(), "top": 64}
 
     def route(self, h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, correction: Optional[torch.Tensor] = None,
-              softmax_all: bool = False) -> torch.Tensor:
+              softmax_all: bool = False, sigmoid: bool = False, extra_gates: int = 0) -> torch.Tensor:
         """Float32 ``[T, experts]``: for every row its weight for each expert, the softmax over the ``top`` largest of the
         logits ``h @ w.T + bias`` (32-bit sums, float32 weights; the lower index wins a tie), zero for the others.  With
         ``softmax_all`` the scores are the softmax over all logits, the ``top`` largest of score + ``correction`` are chosen,
-        and the weights are the chosen scores over their sum (+ 1e-20)."""
+        and the weights are the chosen scores over their sum (+ 1e-20).  With ``sigmoid`` the weights are the sigmoids of the
+        chosen logits.  ``extra_gates``: that many last rows of ``w`` are no experts but gates of every row, the sigmoids of
+        their logits, left in the last columns (``[T, experts + extra_gates]``)."""
         lib = self._extra_lib("routed")
         T, d = h.shape
-        E = w.shape[0]
+        E = w.shape[0] - extra_gates
         self._want(h, self.dtype, "route rows")
-        self._want(w, torch.float32, "route weight", E, d)
+        self._want(w, torch.float32, "route weight", E + extra_gates, d)
         if bias is not None:
             self._want(bias, torch.float32, "route bias", E)
         if correction is not None:
             self._want(correction, torch.float32, "route correction", E)
-        gates = torch.empty((T, E), dtype=torch.float32, device=h.device)
+        gates = torch.empty((T, E + extra_gates), dtype=torch.float32, device=h.device)
         self._check(lib, lib.ms_route(_ptr(h), _ptr(w), _ptr(bias), _ptr(gates), _c_int(T), _c_int(d), _c_int(E), _c_int(top),
-                                      _c_int(int(softmax_all)), _ptr(correction), self._stream()))
+                                      _c_int(1 if softmax_all else (2 if sigmoid else 0)), _ptr(correction), _c_int(extra_gates), self._stream()))
         return gates
 
     def expert_act(self, up: torch.Tensor, gates: torch.Tensor, ff: int, activation: str, experts: Optional[int] = None,
-                   gated: bool = False) -> torch.Tensor:
+                   gated: bool = False, weigh_input: bool = False, shared_gate: bool = False) -> torch.Tensor:
         """``act(up[t, c]) * gates[t, c // ff]`` in the element type for float32 ``up [T, n]``; the columns beyond
         ``experts * ff`` (an expert every row uses) carry weight one.  ``experts``: how many of the gates' columns are
         experts with columns here (None: all).  ``gated``: ``up`` is ``[T, 2 n]``, the experts' gates and then their up
-        projections, and the result ``act(gate) * up * weight``."""
+        projections, and the result ``act(gate) * up * weight``, or with ``weigh_input`` ``act(weight gate) * (weight up)`` for the
+        experts' columns.  ``shared_gate``: the columns beyond the experts carry ``gates[t, experts]`` instead of one."""
         lib = self._extra_lib("routed")
         T, n = up.shape
         if gated:
@@ -1276,7 +1338,8 @@ class HipOps:
             raise KernelError(f"experts: activation {activation!r} is not built (built: {', '.join(sorted(self.EXPERT_ACTIVATIONS))})")
         out = torch.empty((T, n), dtype=self.dtype, device=up.device)
         self._check(lib, lib.ms_expert_act(_ptr(up), _ptr(gates), _ptr(out), _c_int(T), _c_int(n), _c_int(E), _c_int(ff),
-                                           _c_int(self.EXPERT_ACTIVATIONS[activation]), _c_int(gates.shape[1]), _c_int(int(gated)), self._stream()))
+                                           _c_int(self.EXPERT_ACTIVATIONS[activation]), _c_int(gates.shape[1]), _c_int(int(gated)),
+                                           _c_int(int(weigh_input)), _c_int(int(shared_gate)), self._stream()))
         return out
 
     def add_scaled_rows(self, x: torch.Tensor, h: torch.Tensor, weights: torch.Tensor, first: int, count: int) -> None:
@@ -1470,6 +1533,8 @@ class HipOps:
 # The activations a gated product applies to its gate branch, by the name a specification gives them, and the
 # number the kernels know them by.
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+# ... and those of a feed-forward without a gate branch ("relu2": the square of relu).
+UNARY_ACTIVATIONS = {"relu2": 0, "silu": 1, "gelu_tanh": 2}
 
 
 def gate_activation_code(name: str) -> int:

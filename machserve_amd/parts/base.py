@@ -118,10 +118,11 @@ class ResidualStream:
         self.ops = ops
         self.deferred = None                         # (a, w): x += a @ w.T, not yet launched
         self.pending: Optional[torch.Tensor] = None  # float32 [P, T, width], not yet added
+        self.rounded: Optional[torch.Tensor] = None  # x in the element type, if whoever wrote x left it as well
 
     def add_linear(self, a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
         """``x += a @ w.T (+ bias)``."""
-        self.flush()
+        self.open()
         if bias is not None:
             self.x += bias
         self.deferred = (a, w)
@@ -129,19 +130,19 @@ class ResidualStream:
     def add_normed_mean(self, branches, eps: float) -> None:
         """``x += mean_i rmsnorm(a_i @ w_i.T) * g_i`` for branches side by side, each given as ``((a, w), g)``: the
         operands of its last product and the weight of its norm."""
-        self.flush()
+        self.open()
         for (a, w), g in branches:
             self.ops.norm_add(self.x, self.ops.linear_split(a, w), g / float(len(branches)), eps)
 
     def add(self, y: torch.Tensor) -> None:
         """``x += y`` for a part that computes its output by other means."""
-        self.flush()
+        self.open()
         self.x += y.to(self.x.dtype)
 
     def add_rows_scaled(self, h: torch.Tensor, weights: torch.Tensor, first: int, count: int) -> None:
         """``x[t] += (sum of weights[t, first : first + count]) * h[t]``: a part's input itself, weighted row by row (experts
         that return their input).  Comes after the part's ``add_linear``, if it has one."""
-        self.flush()
+        self.open()
         self.ops.add_scaled_rows(self.x, h, weights, first, count)
 
     def launch_deferred(self) -> None:
@@ -157,9 +158,21 @@ class ResidualStream:
             self.ops.add_partials(self.x, self.pending)
             self.pending = None
 
+    def open(self) -> torch.Tensor:
+        """The stream with everything added, about to be written by the caller."""
+        self.flush()
+        self.rounded = None
+        return self.x
+
     def value(self) -> torch.Tensor:
         self.flush()
         return self.x
+
+    def rows(self) -> torch.Tensor:
+        """The stream in the element type, the input of a part that reads it as it is; what the last writer left beside
+        the stream if it did, else rounded here."""
+        x = self.value()
+        return self.rounded if self.rounded is not None else self.ops.round_rows(x)
 
 
 class MultiStream:

@@ -1,4 +1,5 @@
-"""Arrangements of parts in a block.  Post-norm: the branches read the stream itself and are normed on their way out,
+"""Arrangements of parts in a block.  Sum-norm: the norms come after the sums, ``x <- norm(alpha x + mixer(x)); x <- norm(alpha x +
+feed_forward(x))``.  Post-norm: the branches read the stream itself and are normed on their way out,
 ``x += post(mixer(x)); x += post(feed_forward(x))``.  Parallel: one norm feeds both branches, ``x += mixer(norm(x)) + feed_forward(norm(x))``.
 Multi-stream: pre-norm over several residual streams, a branch reading ``sum_s in[s] x_s`` and written back as
 ``x_t = sum_s mix[s, t] x_s + out[t] y``.  Sandwich: a norm before and one after each branch,
@@ -218,11 +219,50 @@ class PostNormBlock(Block):
 
     def _branch(self, part, post, stream, ctx):
         out = _Branch(self.rt.ops)
-        x = stream.value()
-        part.forward(x if getattr(part, "reads_stream", False) else self.rt.ops.round_rows(x), out, ctx)
+        part.forward(stream.value() if getattr(part, "reads_stream", False) else stream.rows(), out, ctx)
         if out.branches is not None:
             post.add_normed_mean(stream, *out.branches)
         elif out.product is not None:
             post.add_normed(stream, *out.product, bias=out.bias)
         else:
             post.add_normed_tensor(stream, out.tensor)
+
+
+@register_block("sumnorm")
+class SumNormBlock(Block):
+    """Reads ``mixer``, ``feed_forward`` (may be None), ``mixer_norm``, ``feed_forward_norm`` and ``alpha`` of its layer's spec.  A
+    branch reads the stream's rows as they are (in the element type, or the 32-bit rows if it says ``reads_stream``); what
+    it leaves is added to ``alpha`` times the stream and the sum is normed, by one kernel that leaves the rows for the
+    next branch as well (a norm with ``normalise_sum``)."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.alpha = float(spec.alpha)
+        self.mixer = MIXERS.build(spec.mixer, rt)
+        self.mixer_norm = NORMS.build(spec.mixer_norm, rt)
+        self.feed_forward = self.feed_forward_norm = None
+        if spec.feed_forward is not None:
+            self.feed_forward = FEED_FORWARDS.build(spec.feed_forward, rt)
+            self.feed_forward_norm = NORMS.build(spec.feed_forward_norm, rt)
+
+    def parts(self):
+        return [self.mixer, self.mixer_norm] + ([self.feed_forward, self.feed_forward_norm] if self.feed_forward is not None else [])
+
+    def forward(self, stream, ctx):
+        self._branch(self.mixer, self.mixer_norm, stream, ctx)
+        if self.feed_forward is not None:
+            self._branch(self.feed_forward, self.feed_forward_norm, stream, ctx)
+
+    def _branch(self, part, norm, stream, ctx):
+        ops = self.rt.ops
+        out = _Branch(ops)
+        part.forward(stream.value() if getattr(part, "reads_stream", False) else stream.rows(), out, ctx)
+        if out.product is not None:
+            sums = ops.linear_split(*out.product)
+        elif out.tensor is not None:
+            sums = out.tensor.float().contiguous().unsqueeze(0)
+        else:
+            raise ValueError(f"{type(part).__name__} left neither a last product nor a finished tensor")
+        if out.scaled is not None:
+            ops.add_scaled_rows(sums[0], *out.scaled)
+        norm.normalise_sum(stream, self.alpha, sums, out.bias)

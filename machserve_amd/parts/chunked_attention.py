@@ -8,6 +8,10 @@ every head, the write of k and v into their pages); the framework's paged attent
 cap as parameters; the output projection.  Keys and values share pools whose heads are as wide as the wider of the
 two, filled with zeros up to the attention tile's size.  The convolution, both norms, the angles and the scores are
 32-bit in every build.
+
+Variants that the spec names: no convolution, cap or biases; norms over each head of q and k by itself; a sink in the
+softmax and a sigmoid gate per head.  Without a convolution or biases q, k, v and the gate are one product whose partial
+sums the row kernel adds up itself.  Rows never look back further than a chunk, so the cache manager keeps a chunk of keys.
 """
 from __future__ import annotations
 
@@ -41,7 +45,12 @@ class ChunkedAttention(Mixer):
         limits = getattr(rt.ops, "conv_rows_limits", None)
         if limits is not None and self.n + self.rot > limits()["row"]:
             raise ValueError(f"chunked_attention: a row of q, k and v of {self.n} numbers; the kernels take up to {limits()['row'] - self.rot}")
-        limits = getattr(rt.ops, "linrec_limits", None)
+        self.head_norm, self.sink, self.head_gate = (bool(getattr(s, n, False)) for n in ("head_norm", "sink", "head_gate"))
+        if self.head_norm and s.qk_norm:
+            raise ValueError("chunked_attention: norms over the whole of q and k and norms over their heads exclude each other")
+        # q, k, v and the gate as one product that leaves its partial sums to the row kernel
+        self.fused = self.head_norm and not self.taps and not s.bias
+        limits = getattr(rt.ops, "linrec_limits", None) if self.taps else None
         if limits is not None and self.taps > limits()["taps"]:
             raise ValueError(f"chunked_attention: {self.taps} taps; the convolution takes up to {limits()['taps']}")
         self.group = self.kpool = self.vpool = self.state = None
@@ -60,23 +69,35 @@ class ChunkedAttention(Mixer):
                 decls.append(TensorDecl(f"{name}.conv", (n, self.taps), "vector"))
         if s.qk_norm:
             decls += [TensorDecl("q.norm", (self.nq,), "vector"), TensorDecl("k.norm", (self.nk,), "vector")]
+        if self.head_norm:
+            decls += [TensorDecl("q.norm", (s.head_dim,), "vector"), TensorDecl("k.norm", (s.head_dim,), "vector")]
+        if self.sink:
+            decls.append(TensorDecl("sink", (s.heads,), "vector"))
+        if self.head_gate:
+            decls.append(TensorDecl("g.weight", (s.heads, s.hidden)))
         decls.append(TensorDecl("o.weight", (s.hidden, s.heads * s.v_head_dim)))
         return decls
 
     def load(self, t):
         s = self.spec
         names = ("q", "k", "v")
+        self.w_gate, self.sinks = t.get("g.weight"), t.get("sink")
         self.w_qkv = torch.cat([t[n + ".weight"] for n in names], dim=0).contiguous()
         self.b_qkv = torch.cat([t[n + ".bias"] for n in names]).contiguous() if s.bias else None
         self.conv_w = torch.cat([t[n + ".conv"] for n in names], dim=0).contiguous() if self.taps else None
-        self.q_norm, self.k_norm = (t["q.norm"], t["k.norm"]) if s.qk_norm else (None, None)
+        if self.fused and self.head_gate:
+            # (rows of zeros behind the gate: the row kernel reads rows of a multiple of 8 numbers in quads)
+            fill = -(self.n + s.heads) % 8
+            self.w_qkv = torch.cat([self.w_qkv, self.w_gate, self.w_gate.new_zeros((fill, s.hidden))], dim=0).contiguous()
+        self.q_norm, self.k_norm = (t["q.norm"], t["k.norm"]) if s.qk_norm or self.head_norm else (None, None)
         w_o = t["o.weight"]
         if self.hd != s.v_head_dim:  # the attention's output has the pools' head size: columns of zeros in between
             w_o = torch.nn.functional.pad(w_o.view(s.hidden, s.heads, s.v_head_dim), (0, self.hd - s.v_head_dim)).reshape(s.hidden, -1)
         self.w_o = w_o.contiguous()
 
     def cache_request(self):
-        pages = PagedKVRequest(self.spec.kv_heads, self.hd, self.spec.window)
+        reach = [r for r in (self.spec.window, self.spec.chunk) if r]
+        pages = PagedKVRequest(self.spec.kv_heads, self.hd, min(reach) if reach else None)
         if self.taps < 2:
             return pages
         return [pages, StateRequest({"conv": (self.taps - 1, self.n)})]
@@ -96,20 +117,30 @@ class ChunkedAttention(Mixer):
         s, ops = self.spec, self.rt.ops
         view = ctx.groups[self.group]
         g = self.attention_rows_per_token()
-        if self.taps:
+        inv_freq = self.position.rotary_inv_freq() if self.position is not None else None
+        if self.fused:
+            rows = ops.linear_split(h, self.w_qkv)
+        elif self.taps:
             rows = ops.conv_sums(ops.linear_split(h, self.w_qkv), 0, self.n, self.b_qkv, self.conv_w, None, self.state,
                                  ctx.seq_q_start, ctx.seq_q_len, ctx.seq_slot)
         else:
             rows = ops.linear(h, self.w_qkv, self.b_qkv, out_f32=True)
-        inv_freq = self.position.rotary_inv_freq() if self.position is not None else None
-        q = ops.finish_rows(rows, self.q_norm, self.k_norm, s.norm_eps, ctx.position_axis(0), inv_freq, self.rot, self.neighbours,
-                            view.slot_map, self.kpool, self.vpool, s.heads, s.kv_heads, s.head_dim, s.v_head_dim, view.page_size)
+        gate = None
+        if self.head_norm:
+            q, gate = ops.finish_heads(rows, self.q_norm, self.k_norm, s.norm_eps, ctx.position_axis(0), inv_freq, self.rot, self.neighbours,
+                                       self.fused and self.head_gate, view.slot_map, self.kpool, self.vpool, s.heads, s.kv_heads,
+                                       s.head_dim, s.v_head_dim, view.page_size)
+        else:
+            q = ops.finish_rows(rows, self.q_norm, self.k_norm, s.norm_eps, ctx.position_axis(0), inv_freq, self.rot, self.neighbours,
+                                view.slot_map, self.kpool, self.vpool, s.heads, s.kv_heads, s.head_dim, s.v_head_dim, view.page_size)
+        if self.head_gate and gate is None:
+            gate = ops.sigmoid_rows(ops.linear(h, self.w_gate, None, out_f32=True))
         chunk, cap = int(s.chunk or 0), float(s.softcap or 0.0)
         if ctx.decode_only and g <= ops.DECODE_MAX_GROUP:
             o = ops.decode_attention(q, self.kpool, self.vpool, view.block_table, ctx.seq_pos0, s.heads, s.kv_heads, self.hd,
-                                     view.page_size, s.window, float(s.scale), chunk=chunk, softcap=cap)
+                                     view.page_size, s.window, float(s.scale), sinks=self.sinks, out_gate=gate, chunk=chunk, softcap=cap)
         else:
             o = ops.paged_attention(q, self.kpool, self.vpool, view.block_table, ctx.seq_q_start, ctx.seq_q_len, ctx.seq_pos0,
                                     ctx.attention_work[g], s.heads, s.kv_heads, self.hd, view.page_size, s.window, float(s.scale),
-                                    chunk=chunk, softcap=cap)
+                                    sinks=self.sinks, out_gate=gate, chunk=chunk, softcap=cap)
         stream.add_linear(o, self.w_o)

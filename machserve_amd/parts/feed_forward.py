@@ -4,12 +4,13 @@ the tanh form of GELU: ``crates/mach-model/src/kernels.rs:199-208``).  Which act
 specification's to say.  Gate and up are one product whose epilogue applies the activation; down
 accumulates into the 32-bit stream.  With biases on every projection the gate/up product leaves 32-bit sums, a small kernel
 adds the biases' effect (they ride in the product's epilogue), applies the activation and multiplies, and the down
-projection's bias goes into the stream with its product."""
+projection's bias goes into the stream with its product.  Beside it the plain feed-forward without a gate branch,
+``down(act(up(x)))``, whose activation is the up product's epilogue."""
 from __future__ import annotations
 
 import torch
 
-from ..kernels.ops import GATE_ACTIVATIONS, interleave_gate_up
+from ..kernels.ops import GATE_ACTIVATIONS, UNARY_ACTIVATIONS, interleave_gate_up
 from .base import FeedForward, PendingNorm, TensorDecl, require_kernel_sizes
 from .registry import register_feed_forward
 
@@ -55,3 +56,29 @@ class GatedMlp(FeedForward):
         else:
             a = self.rt.ops.linear_swiglu(h, self.w_gate_up, self.spec.intermediate, self.spec.activation)
         stream.add_linear(a, self.w_down)
+
+
+@register_feed_forward("plain_mlp")
+class PlainMlp(FeedForward):
+    """``down(act(up(x)))``; the joint size is filled up with zeros to a multiple of 8, which every activation built maps to zeros."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        if spec.activation not in UNARY_ACTIVATIONS:
+            raise ValueError(f"plain_mlp: activation {spec.activation!r} is not built (built: {', '.join(sorted(UNARY_ACTIVATIONS))})")
+        require_kernel_sizes(rt, "plain_mlp", [("hidden size", spec.hidden)])
+
+    def tensor_decls(self):
+        s = self.spec
+        return [TensorDecl("up.weight", (s.intermediate, s.hidden)), TensorDecl("down.weight", (s.hidden, s.intermediate))]
+
+    def load(self, t):
+        fill = -self.spec.intermediate % 8
+        pad = torch.nn.functional.pad
+        self.w_up = pad(t["up.weight"], (0, 0, 0, fill)).contiguous()
+        self.w_down = pad(t["down.weight"], (0, fill)).contiguous()
+
+    def forward(self, h, stream, ctx):
+        if isinstance(h, PendingNorm):
+            h = h.tensor()
+        stream.add_linear(self.rt.ops.linear_act(h, self.w_up, self.spec.activation), self.w_down)

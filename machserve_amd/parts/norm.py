@@ -44,7 +44,7 @@ class RMSNorm(Norm):
     def add_normed(self, stream, a, w, bias=None) -> None:
         """``x += rmsnorm(a @ w.T (+ bias)) * weight``: the norm after a branch whose last step is a product.  The product
         leaves its sums in 32-bit, and one kernel adds them up, normalises the row and adds it to the stream."""
-        stream.flush()
+        stream.open()
         if bias is None:
             stream.ops.norm_add(stream.x, stream.ops.linear_split(a, w), self.weight, self.spec.eps)
         else:
@@ -58,13 +58,20 @@ class RMSNorm(Norm):
         ((a, w_a), wa), ((b, w_b), wb) = branches
         if eps != self.spec.eps:
             raise ValueError(f"branches normed with eps {eps} under a norm with eps {self.spec.eps}")
-        stream.flush()
+        stream.open()
         ops = stream.ops
         ops.pair_norm_add(stream.x, ops.linear_split(a, w_a), wa, ops.linear_split(b, w_b), wb, self.weight, self.spec.eps)
 
+    def normalise_sum(self, stream, alpha: float, sums, bias=None) -> None:
+        """``x <- rmsnorm(alpha x + sum(sums) (+ bias)) * weight``: the norm behind a residual sum.  ``sums`` float32 ``[P, T,
+        width]`` are what a branch's last product left; one kernel adds them up, normalises the row and leaves it in
+        32-bit and in the element type, which is what the next branch reads."""
+        x = stream.open()
+        stream.rounded = stream.ops.sum_norm(x, sums, bias, alpha, self.weight, self.spec.eps)
+
     def add_normed_tensor(self, stream, y) -> None:
         """``x += rmsnorm(y) * weight`` for a branch that computes its output by other means."""
-        stream.flush()
+        stream.open()
         stream.ops.norm_add(stream.x, y.float().contiguous().unsqueeze(0), self.weight, self.spec.eps)
 
 

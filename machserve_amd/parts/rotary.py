@@ -1,7 +1,7 @@
 """Rotary position encoding with the rotate-half pairing ``(j, j + head_dim/2)`` and
 ``freq_j = theta^(-2j/head_dim)`` (``crates/mach-model/src/kernels.rs:589-660``,
 ``crates/mach-model/src/ref_model.rs:669-704``), optionally with YaRN's scaled frequencies
-(``crates/mach-model/src/ref_model.rs:636-667``).  The table of inverse frequencies is made
+(``crates/mach-model/src/ref_model.rs:636-667``) or with frequencies scaled by their wavelength.  The table of inverse frequencies is made
 once, in 32-bit; the angle ``pos * freq`` and its sine and cosine are computed in 32-bit by
 the kernel that also writes the cache."""
 from __future__ import annotations
@@ -52,6 +52,14 @@ class Rotary(PositionEncoding):
             inv = (1.0 / (f32(yarn.factor) * torch.pow(theta, 2.0 * j / hd))) * ramp + inv * (1.0 - ramp)
             ln = math.log(yarn.factor)
             self.factor = (0.1 * yarn.mscale * ln + 1.0) / (0.1 * yarn.mscale_all_dim * ln + 1.0)
+        bands = getattr(spec, "wavelengths", None)
+        if bands is not None:
+            # `turns`: how often a pair turns within the original context.  Above `high` turns a frequency stays, below `low`
+            # it is divided by the factor, and in between it goes over from one to the other in proportion.
+            turns = bands.original * inv / (2.0 * math.pi)
+            s = (turns - bands.low) / (bands.high - bands.low)
+            mixed = (1.0 - s) * inv / bands.factor + s * inv
+            inv = torch.where(turns > bands.high, inv, torch.where(turns < bands.low, inv / bands.factor, mixed))
         inv = inv.to(torch.float32)
         key = (str(rt.device), inv.numpy().tobytes())
         table = _TABLES.get(key)

@@ -92,6 +92,10 @@ class EmulatedOps:
         up = a.float() @ w[:, 1].reshape(Ip, -1).t()
         return self._r((_act(gate, activation) * up)[:, :intermediate])
 
+    def linear_act(self, a, w, activation):
+        y = a.float() @ w.float().t()
+        return self._r(torch.relu(y) ** 2 if activation == "relu2" else _act(y, activation))
+
     def rope_kv_write(self, qkv, bias, positions, inv_freq, slot_map, kpool, vpool, H, KV, hd, page_size):
         qkv = qkv if qkv.dim() == 2 else qkv.sum(0)
         if bias is not None:
@@ -308,6 +312,11 @@ class EmulatedOps:
         y = partials.sum(0) + (bias if bias is not None else 0.0)
         x += y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps)) * weight
 
+    def sum_norm(self, x, partials, bias, alpha, weight, eps):
+        v = alpha * x + partials.sum(0) + (bias if bias is not None else 0.0)
+        x.copy_(v * (1.0 / torch.sqrt((v * v).sum(-1, keepdim=True) / v.shape[-1] + eps)) * weight)
+        return x if self.dtype == torch.float32 else self._r(x)
+
     def pair_norm_add(self, x, pa, wa, pb, wb, weight, eps):
         rms = lambda y: y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps))
         x += rms(0.5 * (rms(pa.sum(0)) * wa + rms(pb.sum(0)) * wb)) * weight
@@ -366,6 +375,20 @@ class EmulatedOps:
         qo = torch.zeros(T, H, dp)
         qo[..., :d] = q
         return self._r(qo).view(T, H * dp)
+
+    def finish_heads(self, proj, q_norm, k_norm, eps, positions, inv_freq, rot, neighbours, gated, slot_map, kpool, vpool, H, KV, d, dv,
+                     page_size):
+        row = proj.sum(0) if proj.dim() == 3 else proj
+        T, nq, nk = row.shape[0], H * d, KV * d
+
+        def normed(x, heads, w):
+            x = x.reshape(T, heads, d)
+            return x if w is None else x * (1.0 / torch.sqrt((x * x).sum(-1, keepdim=True) / d + eps)) * w
+        q, k = normed(row[:, :nq], H, q_norm).reshape(T, nq), normed(row[:, nq:nq + nk], KV, k_norm).reshape(T, nk)
+        rows = torch.cat([q, k, row[:, nq + nk:nq + nk + KV * dv]], 1)
+        qo = self.finish_rows(rows, None, None, eps, positions, inv_freq, rot, neighbours, slot_map, kpool, vpool, H, KV, d, dv, page_size)
+        n = nq + nk + KV * dv
+        return qo, torch.sigmoid(row[:, n:n + H]) if gated else None
 
     # ------------------------------------------------------------------ linear recurrences with gates that depend on the token
     def linrec_limits(self):
@@ -446,8 +469,15 @@ class EmulatedOps:
     def route_limits(self):
         return {"experts": 1024, "top": 64}
 
-    def route(self, h, w, bias, top, correction=None, softmax_all=False):
+    def route(self, h, w, bias, top, correction=None, softmax_all=False, sigmoid=False, extra_gates=0):
         z = h.float() @ w.t()
+        if extra_gates:  # the last rows are no experts but gates of every row
+            z, extra = z[:, :-extra_gates], torch.sigmoid(z[:, -extra_gates:])
+            return torch.cat([self._weights(z, bias, top, correction, softmax_all, sigmoid), extra], 1)
+        return self._weights(z, bias, top, correction, softmax_all, sigmoid)
+
+    @staticmethod
+    def _weights(z, bias, top, correction, softmax_all, sigmoid):
         if bias is not None:
             z = z + bias
         if softmax_all:  # scores over every output; a correction for the choice only; the chosen scores over their sum
@@ -460,24 +490,30 @@ class EmulatedOps:
             return gates
         val, idx = torch.topk(z, top, dim=-1)
         gates = torch.zeros_like(z)
-        gates.scatter_(1, idx, torch.softmax(val, -1))
+        gates.scatter_(1, idx, torch.sigmoid(val) if sigmoid else torch.softmax(val, -1))
         return gates
 
-    def expert_act(self, up, gates, ff, activation, experts=None, gated=False):
+    def expert_act(self, up, gates, ff, activation, experts=None, gated=False, weigh_input=False, shared_gate=False):
         T, n = up.shape
         E = gates.shape[1] if experts is None else experts
         mul = None
         if gated:  # the first half of the columns are the gates, the second the up projections
             n //= 2
             up, mul = up[:, :n], up[:, n:]
+        wgt = torch.ones(T, n)
+        if shared_gate:
+            wgt[:, E * ff:] = gates[:, E:E + 1]
+        wgt[:, :E * ff] = gates[:, :E].repeat_interleave(ff, dim=1)
+        if weigh_input:  # the experts' weights stand inside
+            inner = wgt.clone()
+            inner[:, E * ff:] = 1.0
+            up = up * inner
         if activation == "gelu":
             a = 0.5 * up * (1.0 + torch.erf(up * 0.7071067811865476))
         else:
             a = _act(up, activation)
         if mul is not None:
             a = a * mul
-        wgt = torch.ones(T, n)
-        wgt[:, :E * ff] = gates[:, :E].repeat_interleave(ff, dim=1)
         return self._r(torch.where(wgt != 0, a * wgt, torch.zeros(())))
 
     def add_scaled_rows(self, x, h, weights, first, count):

@@ -179,8 +179,8 @@ def test_a_slot_used_again_starts_every_state_from_zeros(tmp_path):
 
 def test_what_the_layers_ask_of_the_cache(tmp_path):
     lm = loaded(U.make_dir(tmp_path, "mixed", seed=6))
-    # two attention layers with heads of different sizes: two groups of all keys; every layer and the embedding keep a state
-    assert len(lm.cache.groups) == 2 and all(g.spec.window is None for g in lm.cache.groups.values())
+    # two attention layers with chunks of different lengths, each keeping a chunk of keys; every layer and the embedding keep a state
+    assert sorted(g.spec.window for g in lm.cache.groups.values()) == [16, 24]
     states = lm.cache.states
     assert (5, 0) in states and states[(5, 0)].dtype == torch.int32                     # the embedding's previous token
     assert set(states[(1, 0)].shapes) == {"prev", "wkv"} and set(states[(2, 0)].shapes) == {"lru", "conv"}
