@@ -362,6 +362,22 @@ def befirax_configs(z):
     return befirax, melerax, qwen
 
 
+def livovik_configs(z):
+    """(Livovik, Melerax, Qwen2) configurations of one size.  Livovik: chunked attention with norms, sinks and gates per head,
+    chunks as long as the other designs' window, half of every head rotated; a dense feed-forward and routed experts in
+    turn (8 gated experts of half the dense size, 2 a token, and a gated one of that size for every token).  No layer runs
+    another's tensors, so that every layer's weights come from memory as in the other designs."""
+    w, H, kv, hd = z["width"], z["heads"], z["kv"], z["hd"]
+    att = {"heads": H, "kv_heads": kv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": z["window"]},
+           "rot": {"base": 500000.0, "dims": hd // 2, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 1024}}}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"] // 2}, "router": {"experts": 8, "top": 2}, "shared": {"ff": z["ff"] // 2}}
+    layers = [{"type": "attention", "mixer": att, "mlp": {"kind": "dense", "ff": z["ff"]}}, {"type": "attention", "mixer": att, "mlp": moe}]
+    livovik = {"architecture": "Livovik", "vocab": DESIGN_VOCAB, "width": w, "norm": {"eps": 1e-6}, "postln_alpha": 2.0,
+               "layers": layers * (z["layers"] // 2)}
+    melerax, _, qwen = melerax_configs(z)
+    return livovik, melerax, qwen
+
+
 def compare_designs(args) -> int:
     """Prefill (one prompt in one step) and decode (a batch of single tokens at a context, from the captured step)
     of both designs through the step function; random weights, synthetic tokens.  One JSON line."""
@@ -381,6 +397,8 @@ def compare_designs(args) -> int:
             pairs = list(zip(("melerax", "renanex", "qwen2"), melerax_configs(z)))
         elif design == "befirax":
             pairs = list(zip(("befirax", "melerax", "qwen2"), befirax_configs(z)))
+        elif design == "livovik":
+            pairs = list(zip(("livovik", "melerax", "qwen2"), livovik_configs(z)))
         else:
             pairs = list(zip((design, "qwen2"), nubodra_configs(z) if design == "nubodra" else design_configs(z)))
         for name, raw in pairs:
@@ -449,11 +467,12 @@ def main() -> int:
     ap.add_argument("--designs", action="store_true",
                     help="instead of the default run: prefill and decode throughput of Renanex layers (Mamba scan, attention whose heads "
                          "exchange scores over a window, lightning attention) beside Qwen2 layers of equal sizes, at a few sizes")
-    ap.add_argument("--design", default="renanex", choices=["renanex", "nubodra", "melerax", "befirax"],
+    ap.add_argument("--design", default="renanex", choices=["renanex", "nubodra", "melerax", "befirax", "livovik"],
                     help="with --designs: which design stands beside Qwen2 (nubodra: latent attention and attention behind a convolution, "
                          "beside Qwen2 layers that see every key; befirax: state-space duality, differential and latent attention and gated "
                          "experts over two residual streams, beside Melerax and Qwen2; melerax: chunked attention beside a gated linear recurrence, time mixing "
-                         "and routed experts, beside Renanex and Qwen2 layers)")
+                         "and routed experts, beside Renanex and Qwen2 layers; livovik: chunked attention with sinks and gates per head and experts "
+                         "weighed at their inputs under norms behind the sums, beside Melerax and Qwen2 layers)")
     ap.add_argument("--design-sizes", default="small,medium", help="with --designs: which of the sizes to run (small, medium, large)")
     ap.add_argument("--record-calls", default=None, help=argparse.SUPPRESS)  # file that receives one step's operations (the traced run)
     args = ap.parse_args()

@@ -1,0 +1,428 @@
+"""Livovik on the GPU: every new kernel alone against the CPU stand-in of the same entry point (written from the
+mechanisms' equations) or the plain model's function, and the whole engine (cuts of prompts, decoding, mixed batches with
+pages and slots used again, captured steps, generation) against the plain model."""
+import json
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+
+import livovik_util as U
+from emulated_ops import EmulatedOps
+from gpu_util import DEV
+from plain import livovik_plain as P
+
+pytestmark = pytest.mark.gpu
+
+DTYPES = [torch.float32, torch.bfloat16]
+F32 = 1e-4     # float32 against the plain model in 64-bit
+F64 = torch.float64
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+
+def sharpen_for(dtype):
+    """Softmaxes far from flat for the 32-bit runs, where a wrong key must show; milder for bfloat16, whose rounding a
+    sharp softmax multiplies."""
+    return 3.0 if dtype == torch.float32 else 1.5
+
+
+def ops_of(dtype):
+    from machserve_amd.kernels import get_ops
+    return get_ops(dtype, DEV)
+
+
+def dev(t, dtype=None):
+    return None if t is None else t.to(device=DEV, dtype=dtype or t.dtype).contiguous()
+
+
+def i32(values):
+    return torch.tensor(values, dtype=torch.int32)
+
+
+def close(got, want, dtype, what="", scale_by=None):
+    got, want = got.float().cpu().double(), want.double().cpu()
+    bound = (1e-4 if dtype == torch.float32 else 2e-2) * float((scale_by if scale_by is not None else want).abs().max()) + 1e-6
+    err = float((got - want).abs().max())
+    assert err <= bound, f"{what}: error {err:.3e} over {bound:.3e}"
+
+
+# ------------------------------------------------------------------ the norm behind a sum
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d,T", [(48, 5), (130, 37), (1024, 70), (1028, 3), (2048, 9), (4096, 5), (4100, 2), (5120, 3)])
+def test_norm_of_the_scaled_stream_and_a_branch(dtype, d, T):
+    ops, ref = ops_of(dtype), EmulatedOps(dtype)
+    torch.manual_seed(d)
+    w = torch.randn(d)
+    for parts, alpha, bias in ((1, 2.5, None), (2, 0.5, torch.randn(d)), (3, 1.0, None), (8, 1.7, None), (13, -0.3, torch.randn(d)), (17, 2.0, None)):
+        x, sums = torch.randn(T, d) * 3, torch.randn(parts, T, d)
+        want_x = x.clone()
+        want_h = ref.sum_norm(want_x, sums, bias, alpha, w, 1e-5)
+        got_x = dev(x)
+        got_h = ops.sum_norm(got_x, dev(sums), dev(bias), alpha, dev(w), 1e-5)
+        close(got_x, want_x, torch.float32, f"stream after {parts} sums")
+        close(got_h, want_h, dtype, f"rows for the next branch after {parts} sums")
+        assert got_h.dtype == dtype
+
+
+# ------------------------------------------------------------------ a product with the activation in its epilogue
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("M", [1, 7, 16, 33, 64, 65, 300])
+@pytest.mark.parametrize("N,K", [(80, 64), (40, 48), (264, 128), (2056, 520)])
+def test_product_with_the_activation(dtype, M, N, K):
+    ops, ref = ops_of(dtype), EmulatedOps(dtype)
+    torch.manual_seed(M * N)
+    a, w = torch.randn(M, K).to(dtype), (torch.randn(N, K) * K ** -0.5).to(dtype)
+    for act in ("relu2", "silu", "gelu_tanh"):
+        close(ops.linear_act(dev(a), dev(w), act), ref.linear_act(a, w, act), dtype, act)
+
+
+# ------------------------------------------------------------------ rows of q, k, v and gates with norms per head
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,KV,d,dv,rot,neighbours,parts,T", [
+    (4, 2, 16, 24, 8, False, 1, 21), (6, 1, 20, 12, 6, False, 3, 5), (8, 2, 128, 128, 128, False, 1, 70), (8, 2, 128, 64, 64, True, 2, 9),
+    (4, 1, 96, 48, 48, False, 7, 13), (17, 1, 64, 64, 32, False, 8, 4), (3, 3, 40, 10, 16, False, 1, 6), (2, 2, 256, 256, 256, False, 4, 3),
+    (4, 4, 64, 40, 0, False, 9, 8), (5, 5, 24, 24, 12, True, 1, 33), (40, 8, 128, 128, 64, False, 1, 2)])
+@pytest.mark.parametrize("gated", [False, True])
+def test_rows_finished_head_by_head(dtype, H, KV, d, dv, rot, neighbours, parts, T, gated):
+    ops, ref = ops_of(dtype), EmulatedOps(dtype)
+    torch.manual_seed(H * d + rot)
+    ps, dp = 16, -(-max(d, dv) // 16) * 16
+    n = (H + KV) * d + KV * dv + H
+    stride = -(-n // 8) * 8
+    proj, pos = torch.randn(parts, T, stride), torch.randint(0, 900, (T,), dtype=torch.int32)
+    inv = (1000.0 ** (-torch.arange(rot // 2, dtype=torch.float32) * 2 / rot)) if rot else None
+    pages = -(-T // ps) + 2
+    slots = torch.randperm(pages * ps)[:T].int()
+    qn, kn = torch.randn(d), torch.randn(d)
+    for norms in ((qn, kn), (None, None)):
+        kpool, vpool = torch.zeros(pages, KV, ps, dp, dtype=dtype), torch.zeros(pages, KV, dp, ps, dtype=dtype)
+        want, wg = ref.finish_heads(proj, *norms, 1e-5, pos, inv, rot, neighbours, gated, slots, kpool, vpool, H, KV, d, dv, ps)
+        gk, gv = torch.zeros_like(kpool, device=DEV), torch.zeros_like(vpool, device=DEV)
+        got, gg = ops.finish_heads(dev(proj), dev(norms[0]), dev(norms[1]), 1e-5, dev(pos), dev(inv), rot, neighbours, gated, dev(slots), gk, gv,
+                                   H, KV, d, dv, ps)
+        close(got, want, dtype, "queries")
+        close(gk, kpool, dtype, "keys in their pages")
+        close(gv, vpool, dtype, "values in their pages")
+        assert (gg is None) == (not gated)
+        if gated:
+            close(gg, wg, torch.float32, "gates")
+
+
+def test_a_row_without_a_place_in_the_cache_is_not_written():
+    ops = ops_of(torch.bfloat16)
+    proj = torch.randn(1, 2, 64, device=DEV)
+    kpool, vpool = torch.zeros(1, 1, 16, 16, dtype=torch.bfloat16, device=DEV), torch.zeros(1, 1, 16, 16, dtype=torch.bfloat16, device=DEV)
+    ops.finish_heads(proj, None, None, 1e-5, dev(i32([0, 0])), None, 0, False, False, dev(i32([-1, 3])), kpool, vpool, 2, 1, 16, 16, 16)
+    assert float(kpool[0, 0, 3].abs().sum()) > 0 and float(kpool.abs().sum()) == float(kpool[0, 0, 3].abs().sum())
+    assert float(vpool.abs().sum()) == float(vpool[0, 0, :, 3].abs().sum())
+
+
+# ------------------------------------------------------------------ routed experts weighed at their inputs, a gated expert for every token
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("E,top,ff,shared,width", [(6, 2, 24, 40, 64), (3, 3, 8, 8, 48), (7, 1, 20, 12, 48), (32, 4, 32, 64, 128), (5, 3, 16, 0, 64),
+                                                   (66, 64, 8, 24, 64), (4, 1, 6, 10, 40), (1, 1, 16, 0, 32)])
+def test_experts_weighed_at_their_inputs_against_the_plain_feed_forward(dtype, E, top, ff, shared, width):
+    from machserve_amd.config import RoutedMlpSpec
+    from machserve_amd.parts import FEED_FORWARDS, Runtime
+    ops = ops_of(dtype)
+    torch.manual_seed(E * ff + shared)
+    T = 37
+    h = torch.randn(T, width).to(dtype)
+    t = {"router": torch.randn(E, width) * 0.3}
+    for e, f in [(f"e{e}", ff) for e in range(E)] + ([("shared", shared)] if shared else []):
+        for s in ("gate", "up"):
+            t[f"{e}.{s}"] = (torch.randn(f, width) * width ** -0.5).to(dtype).float()
+        t[f"{e}.down"] = (torch.randn(width, f) * f ** -0.5).to(dtype).float()
+    if shared:
+        t["shared.sg"] = torch.randn(1, width) * 0.3
+    mlp = {"router": {"experts": E, "top": top}, "expert": {"ff": ff}, "shared": {"ff": shared} if shared else None}
+    t64 = {k: v.double() for k, v in t.items()}
+    want = P.moe(h.double(), t64, "", mlp)
+    idx, wts = P.route(h.double(), t64, "", top)
+    w_router = torch.cat([t["router"]] + ([t["shared.sg"]] if shared else []))
+    gates = ops.route(dev(h), dev(w_router), None, top, sigmoid=True, extra_gates=int(shared > 0))
+    close(gates[:, :E], torch.zeros(T, E, dtype=F64).scatter_(1, idx, wts), torch.float32, "weights of the chosen experts, zero elsewhere")
+    if shared:
+        close(gates[:, E:], torch.sigmoid(h.double() @ t64["shared.sg"].T), torch.float32, "gate of the expert for every token")
+    # the part itself, as a model runs it
+    part = FEED_FORWARDS.build(RoutedMlpSpec("routed_mlp", width, E, top, ff, "silu", shared, False, {}, gated=True, scoring="sigmoid",
+                                             weigh="input", shared_gate=shared > 0), Runtime(torch.device(DEV), dtype, ops))
+    own = {"router.weight": dev(t["router"]), **{k: dev(v, dtype) for k, v in t.items() if k.endswith((".gate", ".up", ".down"))}}
+    if shared:
+        own["shared.gate_weight"] = dev(t["shared.sg"])
+    assert {d.name for d in part.tensor_decls()} == set(own)
+    part.load(own)
+
+    class Out:
+        def add_linear(self, a, w, bias=None):
+            self.y = ops.linear(a, w, None, out_f32=True)
+    out = Out()
+    part.forward(dev(h), out, None)
+    close(out.y, want, dtype, "the sum of the chosen experts and the gated one")
+
+
+def test_a_gate_of_every_row_goes_with_softmax_weights_too():
+    ops, ref = ops_of(torch.float32), EmulatedOps(torch.float32)
+    torch.manual_seed(0)
+    h, w = torch.randn(9, 32), torch.randn(7, 32)
+    close(ops.route(dev(h), dev(w), None, 2, extra_gates=2), ref.route(h, w, None, 2, extra_gates=2), torch.float32)
+    up, gates = torch.randn(9, 40), torch.rand(9, 6)
+    close(ops.expert_act(dev(up), dev(gates), 6, "gelu", experts=5, shared_gate=True), ref.expert_act(up, gates, 6, "gelu", experts=5, shared_gate=True),
+          torch.float32, "experts without gates beside a gated one for every row")
+
+
+# ------------------------------------------------------------------ attention over chunks with a sink and a gate per head
+def _keys_case(dtype, H, KV, hd, ps, before, now, key, chunk, sinks=None, gate=None, freed=True):
+    """One request with ``before`` keys in the cache and ``now`` rows; key ``key`` is made to stand out for the last row's
+    first head of every group (its value is 50 in every column).  Pages that lie wholly behind the first row's chunk have
+    been given back.  The kernels against the stand-in; returns the last row."""
+    ops, ref = ops_of(dtype), EmulatedOps(dtype)
+    torch.manual_seed(before + now)
+    total = before + now
+    n_pages = -(-total // ps)
+    table = (torch.randperm(n_pages) + 1).int().view(1, -1)
+    kpool, vpool = torch.randn(n_pages + 1, KV, ps, hd).to(dtype), torch.randn(n_pages + 1, KV, hd, ps).to(dtype)
+    q = torch.randn(now, H * hd)
+    page, off = int(table[0, key // ps]), key % ps
+    for kvh in range(KV):
+        h = kvh * (H // KV)
+        kpool[page, kvh, off] = (q[-1, h * hd:(h + 1) * hd] * 4).to(dtype)
+    vpool[page, :, :, off] = 50.0
+    if chunk and freed:
+        table[0, :(before // chunk * chunk) // ps] = -1
+    q = q.to(dtype)
+    g = H // KV
+    unit = ops.attention_rows_per_block(hd)
+    ref.rows_per_block = unit
+    work = torch.tensor([[0, r0] for r0 in range(0, now * g, unit)], dtype=torch.int32)
+    args = (i32([0]), i32([now]), i32([before]))
+    kw = lambda f: dict(sinks=f(sinks), out_gate=f(gate), chunk=chunk)
+    want = ref.paged_attention(q, kpool, vpool, table, *args, work, H, KV, hd, ps, None, 0.5, **kw(lambda t: t))
+    got = ops.paged_attention(dev(q), dev(kpool), dev(vpool), dev(table), *[dev(a) for a in args], dev(work), H, KV, hd, ps, None, 0.5, **kw(dev))
+    close(got, want, dtype, "mixed-batch kernel", scale_by=want.abs().max().clamp(min=1.0))
+    if now == 1 and g <= ops.DECODE_MAX_GROUP:
+        got = ops.decode_attention(dev(q), dev(kpool), dev(vpool), dev(table), dev(args[2]), H, KV, hd, ps, None, 0.5, **kw(dev))
+        close(got, want, dtype, "decode kernel", scale_by=want.abs().max().clamp(min=1.0))
+    return want[-1]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("decoded", [False, True])
+@pytest.mark.parametrize("chunk,n,key,seen", [(136, 800, 680, True), (136, 800, 679, False), (136, 800, 799, True), (136, 816, 680, True), (136, 817, 815, False),
+                                              (20, 300, 280, True), (20, 300, 279, False), (64, 640, 576, True), (64, 640, 575, False), (64, 641, 640, True),
+                                              (7, 50, 49, True), (7, 50, 48, False), (1000, 800, 0, True), (200, 200, 0, True), (200, 201, 0, False),
+                                              (1, 70, 69, True), (1, 70, 68, False), (0, 800, 0, True), (0, 800, 511, True)])
+def test_a_key_that_stands_out_is_seen_only_inside_the_chunk(dtype, decoded, chunk, n, key, seen):
+    """The last row of ``n`` under a gate of a half and a sink too small to matter: the chunk's first position, the one
+    before it, keys at page borders, the first key of all, the row itself."""
+    H, KV, hd = 8, 2, 96
+    rows = 1 if decoded else n
+    last = _keys_case(dtype, H, KV, hd, 16, n - rows, rows, key, chunk, torch.full((H,), -9.0), torch.full((rows, H), 0.5))
+    top = float(last[:hd].min())
+    assert (20.0 < top < 30.0) if seen else top < 10.0   # 50, halved by the gate
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("decoded", [False, True])
+@pytest.mark.parametrize("H,KV,hd", [(8, 2, 96), (17, 1, 32), (4, 4, 64), (4, 1, 128), (3, 3, 240)])
+def test_a_sink_takes_its_share_whatever_the_keys_hold(dtype, decoded, H, KV, hd):
+    """A sink far above every score leaves next to nothing, one far below leaves the softmax as it is, and one per head
+    each takes its own share, under chunks."""
+    n, chunk = 300, 48
+    rows = 1 if decoded else n
+    sinks = torch.linspace(-20.0, 12.0, H)
+    for s, what in ((sinks, "one per head"), (torch.full((H,), 60.0), "far above"), (torch.full((H,), -60.0), "far below")):
+        last = _keys_case(dtype, H, KV, hd, 16, n - rows, rows, 295, chunk, s, torch.rand(rows, H) if what == "one per head" else None)
+        if what == "far above" and hd <= 32:
+            assert float(last[hd:2 * hd].abs().max()) < 1e-3 or H == KV
+
+
+# ------------------------------------------------------------------ the engine against the plain model
+def loaded(model_dir, dtype, page_size=16, max_tokens=1024, max_requests=4, use_graphs=True, num_pages=None):
+    from machserve_amd.engine.loading import load_model
+    return load_model(model_dir, dtype=dtype, device=DEV, page_size=page_size, max_tokens=max_tokens, max_requests=max_requests,
+                      use_graphs=use_graphs, num_pages=num_pages)
+
+
+def _cut(rid, n, sizes):
+    out, at, k = [], 0, 0
+    while at < n:
+        c = min(sizes[k % len(sizes)], n - at)
+        out.append([(rid, c)])
+        at, k = at + c, k + 1
+    return out
+
+
+def plain_for(model_dir, dtype, tokens):
+    """The plain model in 64-bit, on the weights as the run holds them."""
+    return U.plain_logits(model_dir, tokens, torch.float64, weights_as=dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", sorted(U.CONFIGS))
+def test_prompts_cut_anywhere_and_decoding_equal_the_plain_model(tmp_path, name, dtype):
+    d = U.make_dir(tmp_path, name, seed=7, sharpen=sharpen_for(dtype))
+    n = 150
+    toks = U.tokens_of(n, U.CONFIGS[name]["vocab"], 8)
+    want = plain_for(d, dtype, toks)
+    lm = loaded(d, dtype)
+    schedules = {"whole": [[("a", n)]], "prompt, then token by token": [[("a", 60)]] + [[("a", 1)]] * (n - 60),
+                 "portions down to two tokens": _cut("a", n, [2, 33, 3, 16, 2, 47, 1, 1, 31, 2])}
+    for what, schedule in schedules.items():
+        got = U.run_schedule(lm, {"a": toks}, schedule)["a"]
+        assert U.within(got, want, dtype), what
+    lm.cache.check()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_sizes_nearer_a_real_models(tmp_path, dtype):
+    # in bfloat16 the experts stay small beside the stream: with sixteen experts and hundreds of rows some row's choice
+    # sits on a near-tie
+    d = U.make_dir(tmp_path, "big", seed=17, sharpen=1.5, experts=5.0 if dtype == torch.float32 else 2.0)
+    n = 330
+    toks = U.tokens_of(n, 1000, 4)
+    want = plain_for(d, dtype, toks)
+    lm = loaded(d, dtype, page_size=64)
+    for what, schedule in {"whole": [[("a", n)]], "portions, then token by token": _cut("a", 290, [128, 2, 97, 63]) + [[("a", 1)]] * 40}.items():
+        got = U.run_schedule(lm, {"a": toks}, schedule)["a"]
+        assert U.within(got, want, dtype), what
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("graphs", [False, True])
+def test_unequal_requests_side_by_side_equal_each_alone(tmp_path, dtype, graphs):
+    name = "mixed"
+    d = U.make_dir(tmp_path, name, seed=9, sharpen=sharpen_for(dtype))
+    vocab = U.CONFIGS[name]["vocab"]
+    reqs = {"a": U.tokens_of(90, vocab, 1), "b": U.tokens_of(1, vocab, 2), "c": U.tokens_of(41, vocab, 3),
+            "d": U.tokens_of(70, vocab, 4), "e": U.tokens_of(35, vocab, 5)}
+    schedule = [[("b", 1), ("a", 20), ("c", 5)], [("a", 1), ("c", 30)], [("a", 2), ("c", 2), ("d", 17)], [("a", 1), ("c", 1), ("d", 1)],
+                [("a", 1), ("c", 1), ("d", 1)], [("a", 1), ("c", 1), ("d", 1)], [("a", 1), ("c", 1), ("d", 1)],
+                [("d", 1), ("e", 16), ("a", 1)], [("a", 30), ("e", 1), ("d", 2)], [("a", 32), ("d", 46), ("e", 18)]]
+    lm = loaded(d, dtype, max_requests=3, num_pages=16, use_graphs=graphs)
+    got = U.run_schedule(lm, reqs, schedule)
+    for i, toks in reqs.items():
+        assert U.within(got[i], plain_for(d, dtype, toks), dtype), i
+    if dtype == torch.float32:      # and the same numbers, beyond rounding, as each request alone in one step
+        alone = loaded(d, dtype, use_graphs=False)
+        for i, toks in reqs.items():
+            assert U.relative_error(got[i], U.run_schedule(alone, {i: toks}, [[(i, len(toks))]])[i]) < 2e-5, i
+    lm.cache.check()
+    assert all(g.pool.available() == g.pool.num_pages for g in lm.cache.groups.values())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_long_decoding_from_captured_steps(tmp_path, name, dtype):
+    """Decoded tokens pass the edges of many chunks (1, 7, 33 and 32, 100, 200 positions) and leave pages behind; layers
+    that run another's tensors are in the captured steps with caches of their own."""
+    d = U.make_dir(tmp_path, name, seed=10, sharpen=sharpen_for(dtype))
+    toks = U.tokens_of(330, U.CONFIGS[name]["vocab"], 3)
+    lm = loaded(d, dtype, max_tokens=512)
+    got = U.run_schedule(lm, {"a": toks}, [[("a", 10)]] + [[("a", 1)]] * 320)["a"]
+    assert U.within(got, plain_for(d, dtype, toks), dtype)
+    assert len(lm.step._graphs) > 0     # the single rows ran from captured steps
+
+
+def test_a_long_prompt_in_portions_behind_pages_of_64(tmp_path):
+    d = U.make_dir(tmp_path, "mixed", seed=11)
+    toks = U.tokens_of(700, 97, 6)
+    want = plain_for(d, torch.float32, toks)
+    lm = loaded(d, torch.float32, page_size=64, max_tokens=768)
+    for what, schedule in {"whole": [[("a", 700)]], "portions": _cut("a", 700, [500, 63, 2, 129, 6])}.items():
+        got = U.run_schedule(lm, {"a": toks}, schedule)["a"]
+        assert U.relative_error(got, want) < F32, what
+
+
+def test_long_portions_beside_decoded_tokens(tmp_path):
+    d = U.make_dir(tmp_path, "mixed", seed=21)
+    reqs = {"a": U.tokens_of(500, 97, 1), "b": U.tokens_of(320, 97, 2), "c": U.tokens_of(9, 97, 3)}
+    schedule = [[("a", 190), ("b", 200)], [("c", 7), ("b", 118)], [("b", 1), ("a", 305), ("c", 1)], [("b", 1), ("a", 5), ("c", 1)]]
+    lm = loaded(d, torch.float32, page_size=64, max_tokens=1024, max_requests=3)
+    got = U.run_schedule(lm, reqs, schedule)
+    for i, toks in reqs.items():
+        assert U.relative_error(got[i], plain_for(d, torch.float32, toks)) < F32, i
+
+
+def test_first_tokens_of_a_sequence(tmp_path):
+    for name in sorted(U.CONFIGS):
+        d = U.make_dir(tmp_path, name, seed=12)
+        toks = U.tokens_of(4, U.CONFIGS[name]["vocab"], 1)
+        lm = loaded(d, torch.float32)
+        for n in (1, 2, 3, 4):
+            want = plain_for(d, torch.float32, toks[:n])
+            assert U.relative_error(U.run_schedule(lm, {"a": toks[:n]}, [[("a", n)]])["a"], want) < F32, (name, n)
+            assert U.relative_error(U.run_schedule(lm, {"a": toks[:n]}, [[("a", 1)]] * n)["a"], want) < F32, (name, n, "one by one")
+
+
+def test_mistakes_in_the_plain_model_would_show(tmp_path):
+    """The tests' own power: the plain model with a mechanism changed a little is far from what it was."""
+    d = U.make_dir(tmp_path, "mixed", seed=16)
+    toks = U.tokens_of(60, 97, 9)
+    want = plain_for(d, torch.float32, toks)
+    w, cfg = U.read(d)
+
+    def off(change_cfg=None, change_w=None):
+        c, t = json.loads(json.dumps(cfg)), dict(w)
+        if change_cfg:
+            change_cfg(c)
+        if change_w:
+            change_w(t)
+        return U.relative_error(P.forward(t, c, toks, torch.float64)[30:], want[30:])
+
+    def chunks(c):
+        for layer in c["layers"]:
+            if "mask" in layer["mixer"]:
+                layer["mixer"]["mask"]["size"] += 1
+    assert off(chunks) > 1e-2
+    assert off(lambda c: c["layers"][0]["mixer"]["rot"].pop("scaling")) > 1e-3
+    assert off(None, lambda t: t.update({k: v - 30.0 for k, v in t.items() if k.endswith(".sink")})) > 1e-2
+    assert off(None, lambda t: t.update({"l0.mlp.shared.sg": t["l0.mlp.shared.sg"] * 0 + 9.0})) > 1e-2
+    assert off(lambda c: c.update(postln_alpha=1.6)) > 1e-2
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_greedy_generation_through_the_entry_point(tmp_path, dtype):
+    import machserve_amd
+    d = U.make_dir(tmp_path, "mixed", seed=13, sharpen=2.0)
+    w, cfg = U.read(d)
+    prompts = [U.tokens_of(n, 97, n) for n in (3, 21, 1, 40, 17)]
+    got = machserve_amd.generate(d, prompts, max_new=8, dtype=dtype, page_size=16, capacity=3, max_batch_tokens=32, chunk_size=16)
+    for p, g in zip(prompts, got):
+        if dtype == "float32":
+            assert g == P.greedy_generate(w, cfg, p, 8, torch.float64)
+        else:   # bfloat16 may flip a near-tie: every token must be within rounding of the best
+            seq = list(p)
+            for t in g:
+                logits = plain_for(d, torch.bfloat16, seq)[-1]
+                assert logits[t] >= logits.max() - 5e-2 * (logits.max() - logits.min()), "a token that is not a maximum"
+                seq.append(t)
+
+
+def test_a_folder_of_this_layout_runs_through_the_trace_program(tmp_path):
+    import numpy as np
+    d = U.make_dir(tmp_path, "odd", seed=14)
+    toks = U.tokens_of(50, 61, 2)
+    out = tmp_path / "out"
+    steps = [{"step": 0, "entries": [{"id": "x", "tokens": toks[:33], "want": [0, 32]}], "end": []},
+             {"step": 1, "entries": [{"id": "x", "tokens": toks[33:], "want": [16]}, {"id": "y", "tokens": toks[:2], "want": []}], "end": ["x", "y"]}]
+    r = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", d, "--dtype", "float32", "--out", str(out),
+                        "--max-tokens", "128", "--page-size", "16"], input="\n".join(json.dumps(s) for s in steps) + "\n",
+                       capture_output=True, text=True, timeout=600)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [ln for ln in r.stdout.splitlines() if ln.startswith("done")] == ["done 0", "done 1"]
+    want = plain_for(d, torch.float32, toks)
+    got = torch.from_numpy(np.concatenate([np.fromfile(out / "0.f32", dtype="<f4"), np.fromfile(out / "1.f32", dtype="<f4")]).reshape(3, 61))
+    assert U.relative_error(got, want[[0, 32, 49]]) < F32
+
+
+def test_command_line_generates_from_a_folder(tmp_path):
+    d = U.make_dir(tmp_path, "mixed", seed=15)
+    w, cfg = U.read(d)
+    prompt = U.tokens_of(9, 97, 4)
+    cmd = [sys.executable, os.path.join(ROOT, "bin", "machserve"), "--max-new", "5", "--dtype", "f32", "--tpp", "16", "--prompt-ids"]
+    r = subprocess.run(cmd + [",".join(map(str, prompt)), "--model", d], capture_output=True, text=True, timeout=600)
+    assert r.returncode == 0, r.stderr[-2000:]
+    assert [int(t) for t in r.stdout.split()] == P.greedy_generate(w, cfg, prompt, 5, torch.float64)
