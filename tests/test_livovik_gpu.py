@@ -110,6 +110,28 @@ def test_rows_finished_head_by_head(dtype, H, KV, d, dv, rot, neighbours, parts,
             close(gg, wg, torch.float32, "gates")
 
 
+@pytest.mark.parametrize("d,rot", [(64, 64), (20, 6)])
+def test_angles_stay_exact_at_far_positions(d, rot):
+    """Rows at positions up to a hundred thousand against a rotation in 64-bit by the same frequencies: a 32-bit product of
+    position and frequency alone would be off by 4e-3 radians there."""
+    ops = ops_of(torch.float32)
+    torch.manual_seed(d)
+    T, H, ps = 40, 2, 64
+    pos = torch.randint(50000, 100000, (T,), dtype=torch.int32)
+    inv = 100.0 ** (-torch.arange(rot // 2, dtype=torch.float32) * 2 / rot)
+    proj = torch.randn(1, T, -(-(3 * d + 8) // 8) * 8)
+    dp = -(-d // 16) * 16
+    pool = lambda *shape: torch.zeros(*shape, device=DEV)
+    got, _ = ops.finish_heads(dev(proj), None, None, 1e-6, dev(pos), dev(inv), rot, False, False, dev(torch.arange(T, dtype=torch.int32)),
+                              pool(1, 1, ps, dp), pool(1, 1, dp, ps), H, 1, d, 8, ps)
+    q = proj[0, :, :H * d].double().view(T, H, d)
+    a = (pos.double()[:, None] * inv.double())[:, None, :]
+    u, v = q[..., :rot // 2], q[..., rot // 2:rot]
+    want = torch.cat([u * torch.cos(a) - v * torch.sin(a), v * torch.cos(a) + u * torch.sin(a), q[..., rot:]], -1)
+    err = float((got.cpu().double().view(T, H, dp)[..., :d] - want).abs().max())
+    assert err < 2e-5, err
+
+
 def test_a_row_without_a_place_in_the_cache_is_not_written():
     ops = ops_of(torch.bfloat16)
     proj = torch.randn(1, 2, 64, device=DEV)
