@@ -326,10 +326,46 @@ class TimeMixSpec:
 @dataclass(frozen=True)
 class SideBySideSpec:
     """Several mixers that read the same input; each one's output is RMS-normed over the model's width (``norm_eps``) with a
-    weight of its own (``tensors``: ``norm.<i>``), and the result is their mean."""
+    weight of its own (``tensors``: ``norm.<i>``), and the result is their mean.  With ``factors`` (one a branch) there are no such
+    norms, and the result is the sum of the outputs times their factors."""
     kind: str
     hidden: int
     branches: Sequence[object]
+    norm_eps: float = 1e-6
+    tensors: Mapping[str, str] = field(default_factory=dict)
+    factors: Optional[Sequence[float]] = None
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec:
+    """Gated linear attention: ``q = W_q h head_dim^(-1/2)``, ``k = W_k h`` (``heads`` x ``head_dim``), ``v = W_v h`` (``heads`` x ``v_head_dim``); a decay
+    per key channel ``alpha = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau)`` through a bottleneck of ``decay_rank`` (None: whatever the
+    checkpoint's tensors have); per head ``S <- diag(alpha) S + k v^T``, ``o = S^T q``; a head's ``o`` is RMS-normed (``norm_eps``, one weight of
+    ``v_head_dim`` for all heads), the heads side by side are multiplied by ``silu(W_g h)`` and projected."""
+    kind: str
+    hidden: int
+    heads: int
+    head_dim: int
+    v_head_dim: int
+    tau: float = 16.0
+    decay_rank: Optional[int] = None
+    norm_eps: float = 1e-6
+    tensors: Mapping[str, str] = field(default_factory=dict)
+
+
+@dataclass(frozen=True)
+class GatedDeltaSpec:
+    """The gated delta rule: q and k have ``kv_heads`` heads of ``head_dim``, v ``heads`` of ``v_head_dim`` (head h uses q/k head ``h // (heads /
+    kv_heads)``); each passes a causal convolution of ``conv_taps`` per channel and SiLU; q and k of a head become unit vectors
+    (``x / sqrt(sum x^2 + 1e-6)``), q times ``head_dim^(-1/2)``; ``beta = sigmoid(W_b h)``, ``g = exp(-exp(A_log) softplus(W_a h + dt_bias))``
+    per head; ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q``; then as :class:`GatedLinearSpec`."""
+    kind: str
+    hidden: int
+    heads: int
+    kv_heads: int
+    head_dim: int
+    v_head_dim: int
+    conv_taps: int
     norm_eps: float = 1e-6
     tensors: Mapping[str, str] = field(default_factory=dict)
 
@@ -506,6 +542,16 @@ class HeadSpec:
 
 
 @dataclass(frozen=True)
+class LoopStepsSpec:
+    """What comes ahead of each pass over looped layers: ``starts[t]`` is the place in the model's ``order`` where pass t begins.
+    Right before it the stream takes, in every pass but the first, the embedding's output again, and then row t of a table
+    of ``width`` numbers a pass ("step")."""
+    width: int
+    starts: Sequence[int]
+    tensors: Mapping[str, str] = field(default_factory=dict)
+
+
+@dataclass(frozen=True)
 class ModelSpec:
     architecture: str
     embedding: EmbeddingSpec
@@ -516,9 +562,17 @@ class ModelSpec:
     max_positions: int
     # several residual streams, all equal to the embedding at the start and summed at the end (None: the one stream)
     streams: Optional[int] = None
+    # what is added to the stream ahead of each pass over layers that ``order`` runs several times in a row
+    loop_steps: Optional[LoopStepsSpec] = None
 
     def validate(self) -> None:
         n = len(self.layers)
+        if self.loop_steps is not None:
+            if self.streams:
+                raise ConfigError("loop_steps: a model of several residual streams has no passes with steps")
+            starts = list(self.loop_steps.starts)
+            if starts != sorted(set(starts)) or (starts and not 0 <= starts[0] <= starts[-1] < len(self.order)):
+                raise ConfigError(f"loop_steps: the passes begin at {starts} of {len(self.order)} layer runs")
         if not self.order:
             raise ConfigError("order: a model runs at least one layer")
         for i in self.order:

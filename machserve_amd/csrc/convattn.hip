@@ -416,17 +416,6 @@ struct HeadRowArgs {
     int H, KV, d, dv, dp, ps;
 };
 
-// Cosine and sine of position * frequency.  The 32-bit product is off by up to half a unit of its last place, which at a
-// position of a thousand is 3e-5 radians; what it lost is known exactly (one fused multiply-add) and is put
-// back to first order, so that the angle's error does not grow with the position.
-__device__ __forceinline__ void angle_cos_sin(int position, float freq, float& c, float& s) {
-    const float p = (float)position, a = p * freq, rest = __builtin_fmaf(p, freq, -a);
-    float c0, s0;
-    sincosf(a, &s0, &c0);
-    c = c0 - rest * s0;
-    s = s0 + rest * c0;
-}
-
 // Any sizes: the row lies in LDS, a wave sums a head's squares.
 __global__ __launch_bounds__(256) void head_row_kernel(HeadRowArgs a) {
     extern __shared__ float lds[];

@@ -192,38 +192,52 @@ __global__ __launch_bounds__(256) void add_partials_kernel(float* __restrict__ x
 
 // x[t, :] += y / sqrt(mean(y^2) + eps) * w with y = sum_p partials[p, t, :] (in order): a branch's output, given as
 // the partial sums of its last product, normalised and added to the stream in one pass.
-// With `bias` (or null) y also holds a bias of the product, added after the sums.
+// With `bias` (or null) y also holds a bias of the product, added after the sums.  PAIR: two branches side by side,
+// y = fa sum_p partials[p, t, :] + fb sum_p pb[p, t, :] (no bias).
+template <bool PAIR>
 __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, const float* __restrict__ partials, int n_partials,
                                                        size_t partial_stride, const float* __restrict__ w, int d, float eps,
-                                                       const float* __restrict__ bias) {
+                                                       const float* __restrict__ bias, float fa, const float* __restrict__ pb, int nb,
+                                                       float fb) {
     __shared__ float scratch[4];
     extern __shared__ float vals[];  // d floats: the summed row
     const size_t r = blockIdx.x;
     float ss = 0.f;
+    // four columns at c: up to eight sums asked for at once, added in order
+    auto sum4 = [&](const float* __restrict__ from, int n, int c) {
+        const float* src = from + r * d + c;
+        f32x4 v = (f32x4){0.f, 0.f, 0.f, 0.f};
+        int p = 0;
+        for (; p + 8 <= n; p += 8) {
+            f32x4 q[8];
+#pragma unroll
+            for (int k = 0; k < 8; ++k) q[k] = *reinterpret_cast<const f32x4*>(src + (size_t)(p + k) * partial_stride);
+#pragma unroll
+            for (int k = 0; k < 8; ++k) v += q[k];
+        }
+        for (; p < n; ++p) v += *reinterpret_cast<const f32x4*>(src + (size_t)p * partial_stride);
+        return v;
+    };
     if (d % 4 == 0 && partial_stride % 4 == 0) {
-        // four columns a thread and up to eight sums asked for at once, added in order: few trips to memory a row
+        // few trips to memory a row
         for (int c = threadIdx.x * 4; c < d; c += 1024) {
-            const float* src = partials + r * d + c;
-            f32x4 v = (f32x4){0.f, 0.f, 0.f, 0.f};
-            int p = 0;
-            for (; p + 8 <= n_partials; p += 8) {
-                f32x4 q[8];
-#pragma unroll
-                for (int k = 0; k < 8; ++k) q[k] = *reinterpret_cast<const f32x4*>(src + (size_t)(p + k) * partial_stride);
-#pragma unroll
-                for (int k = 0; k < 8; ++k) v += q[k];
-            }
-            for (; p < n_partials; ++p) v += *reinterpret_cast<const f32x4*>(src + (size_t)p * partial_stride);
-            if (bias) v += *reinterpret_cast<const f32x4*>(bias + c);
+            f32x4 v = sum4(partials, n_partials, c);
+            if constexpr (PAIR) v = v * fa + sum4(pb, nb, c) * fb;
+            else if (bias) v += *reinterpret_cast<const f32x4*>(bias + c);
             *reinterpret_cast<f32x4*>(vals + c) = v;
             ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
         }
     } else {
         for (int c = threadIdx.x; c < d; c += 256) {
-            const float* src = partials + r * d + c;
             float v = 0.f;
-            for (int p = 0; p < n_partials; ++p) v += src[(size_t)p * partial_stride];
-            if (bias) v += bias[c];
+            for (int p = 0; p < n_partials; ++p) v += partials[(size_t)p * partial_stride + r * d + c];
+            if constexpr (PAIR) {
+                float b = 0.f;
+                for (int p = 0; p < nb; ++p) b += pb[(size_t)p * partial_stride + r * d + c];
+                v = v * fa + b * fb;
+            } else if (bias) {
+                v += bias[c];
+            }
             vals[c] = v;
             ss += v * v;
         }
@@ -232,6 +246,16 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, co
     const float inv = 1.0f / sqrtf(ss / (float)d + eps);
     float* dst = x + r * d;
     for (int c = threadIdx.x; c < d; c += 256) dst[c] += vals[c] * inv * w[c];
+}
+
+// x[t, :] += first[t, :] (null: nothing) + row: what comes ahead of a pass over looped layers
+__global__ __launch_bounds__(256) void open_pass_kernel(float* __restrict__ x, const float* __restrict__ first, const float* __restrict__ row,
+                                                        int d, size_t n) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    float v = x[i];
+    if (first) v += first[i];
+    x[i] = v + row[i % d];
 }
 
 // x[t, :] = v / sqrt(mean(v^2) + eps) * w with v = alpha * x[t, :] + sum_p partials[p, t, :] (in order) + bias: the norm that
@@ -666,8 +690,8 @@ extern "C" int ms_norm_add(float* x, const float* partials, int n_partials, cons
     MS_REQUIRE(T > 0 && d > 0 && n_partials > 0, "norm_add: empty problem T=%d d=%d with %d sums", T, d, n_partials);
     MS_REQUIRE(d <= MAX_ROW_FLOATS, "norm_add: width %d exceeds the row buffer of %d", d, MAX_ROW_FLOATS);
     MS_REQUIRE(x && partials && w, "norm_add: a buffer is missing");
-    hipLaunchKernelGGL(norm_add_kernel, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, (size_t)T * d, w,
-                       d, eps, (const float*)nullptr);
+    hipLaunchKernelGGL(norm_add_kernel<false>, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, (size_t)T * d, w,
+                       d, eps, (const float*)nullptr, 1.f, (const float*)nullptr, 0, 0.f);
     return check_launch("norm_add");
 }
 
@@ -676,9 +700,27 @@ extern "C" int ms_norm_add_bias(float* x, const float* partials, int n_partials,
     MS_REQUIRE(T > 0 && d > 0 && n_partials > 0, "norm_add: empty problem T=%d d=%d with %d sums", T, d, n_partials);
     MS_REQUIRE(d <= MAX_ROW_FLOATS, "norm_add: width %d exceeds the row buffer of %d", d, MAX_ROW_FLOATS);
     MS_REQUIRE(x && partials && w, "norm_add: a buffer is missing");
-    hipLaunchKernelGGL(norm_add_kernel, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, (size_t)T * d, w,
-                       d, eps, bias);
+    hipLaunchKernelGGL(norm_add_kernel<false>, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, partials, n_partials, (size_t)T * d, w,
+                       d, eps, bias, 1.f, (const float*)nullptr, 0, 0.f);
     return check_launch("norm_add");
+}
+
+// x += rmsnorm(fa sum(pa) + fb sum(pb)) * w
+extern "C" int ms_norm_add_weighted(float* x, const float* pa, int na, float fa, const float* pb, int nb, float fb, const float* w, int T, int d,
+                                    float eps, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && d > 0 && na > 0 && nb > 0, "norm_add_weighted: empty problem T=%d d=%d with %d and %d sums", T, d, na, nb);
+    MS_REQUIRE(d <= MAX_ROW_FLOATS, "norm_add_weighted: width %d exceeds the row buffer of %d", d, MAX_ROW_FLOATS);
+    MS_REQUIRE(x && pa && pb && w, "norm_add_weighted: a buffer is missing");
+    hipLaunchKernelGGL(norm_add_kernel<true>, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, pa, na, (size_t)T * d, w, d, eps,
+                       (const float*)nullptr, fa, pb, nb, fb);
+    return check_launch("norm_add_weighted");
+}
+
+extern "C" int ms_open_pass(float* x, const float* first, const float* row, int T, int d, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && d > 0 && x && row, "open_pass: empty problem T=%d d=%d", T, d);
+    const size_t n = (size_t)T * d;
+    hipLaunchKernelGGL(open_pass_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, first, row, d, n);
+    return check_launch("open_pass");
 }
 
 // x [T, d] <- rmsnorm(alpha x + sum of partials [n_partials, T, d] + bias) * w; out [T, d] in the element type, or null.

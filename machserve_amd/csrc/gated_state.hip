@@ -1,0 +1,1092 @@
+// Linear attention whose memory is a matrix per head, S [d (key channel), dv (value channel)], under gates that depend on
+// the token: gated linear attention (a decay per key channel) and the gated delta rule (a decay per head, and a write that
+// first takes away what the state already holds for the key).
+//
+//   gated linear:  S <- diag(alpha) S + k v^T,                                          o = S^T q
+//   delta rule:    S <- g S;  u = beta (v - S^T k);  S <- S + k u^T,                    o = S^T q
+//
+// Behind both, in the kernel that makes o: a head's o is divided by its root mean square over dv, times one weight for all
+// heads, times silu of a gate, rounded to the element type for the output projection.
+//
+// A step's rows are the tokens of several requests, each request's rows contiguous and in order (seq_q_start, seq_q_len); a
+// request's state lives in slot seq_slot[s] of [slots, H, d, dvp] 32-bit floats (dvp: dv filled up to a multiple of 4 with
+// zeros) and is read at the start of the request's rows and written back after its last.
+//   single rows (decoding)      a block a request and head; the state is read, changed and written once
+//   gated linear, many rows     a thread a value channel with its column of S in registers, token after token; long portions
+//                               in segments side by side (each from zero, then the states between them, then each from its own)
+//   delta rule, many rows       chunks of 64 tokens as small matrix products (below)
+// Decays, their logarithms, step sizes, unit norms, states and every sum and product here are 32-bit in every build; what a
+// token gets depends on the cut of its prompt by rounding only, and on nothing else the step holds.
+#include "recurrence.cuh"
+
+namespace ms {
+
+// Rows given as partial sums [n, T, ld]: a projection's output whose parts the reader adds up.
+struct Sums {
+    const float* p;
+    int n;
+    size_t stride;
+    int ld;
+};
+__device__ __forceinline__ float sum_at(const Sums& a, int t, int c) {
+    const float* src = a.p + (size_t)t * a.ld + c;
+    float v = 0.f;
+#pragma unroll 8
+    for (int i = 0; i < a.n; ++i) v += src[i * a.stride];
+    return v;
+}
+
+constexpr int MAX_TAPS = 16;
+constexpr int MAX_DIM = 256;
+
+// ---- the delta rule's rows: convolution, unit norms, step sizes and decays -----------------------------------
+// in: q [G, d], k [G, d], v [H, dv], gate [H, dv], then at b_col and a_col one number a head each.  On every channel of q, k
+// and v a causal convolution over time (w [C, taps], last tap the current row; earlier inputs from state [slots, taps - 1, C],
+// oldest first) and SiLU; q and k of a head divided by sqrt(sum of squares + 1e-6), q times q_scale; beta = sigmoid(b);
+// lg = -exp(a_log) softplus(a + dt_bias), the logarithm of the head's decay.
+struct DeltaRowsArgs {
+    Sums in;
+    const float* w;
+    float* state;
+    const float* a_log;    // [H]
+    const float* dt_bias;  // [H]
+    const int* seq_q_start;
+    const int* seq_q_len;
+    const int* seq_slot;
+    int S;
+    float* q;     // [T, G * d]
+    float* k;     // [T, G * d]
+    float* v;     // [T, H * dv]
+    float* beta;  // [T, H]
+    float* lg;    // [T, H]
+    int T, H, G, d, dv, taps, b_col, a_col;
+    float q_scale;
+};
+constexpr float UNIT_EPS = 1e-6f;
+
+// A wave takes one head of q, k or v (or the step sizes and decays) over ROWS rows; a lane EPL of its channels, whose last
+// inputs it keeps, so that every input is read once (and again at the start of a block's rows).  A request with a single
+// row gets its state brought up to date here: nobody else reads it.
+template <int TAPS, int EPL, int ROWS>
+__global__ __launch_bounds__(256) void delta_rows_kernel(DeltaRowsArgs a) {
+    const int lane = threadIdx.x & 63, unit = blockIdx.y * 4 + (threadIdx.x >> 6);
+    const int t0 = blockIdx.x * ROWS;
+    if (unit > 2 * a.G + a.H) return;
+    if (unit == 2 * a.G + a.H) {
+        for (int r = 0; r < ROWS && t0 + r < a.T; ++r)
+            for (int h = lane; h < a.H; h += 64) {
+                const int t = t0 + r;
+                a.beta[(size_t)t * a.H + h] = sigmoid_f(sum_at(a.in, t, a.b_col + h));
+                a.lg[(size_t)t * a.H + h] = -expf(a.a_log[h]) * softplus_f(sum_at(a.in, t, a.a_col + h) + a.dt_bias[h]);
+            }
+        return;
+    }
+    const bool is_v = unit >= 2 * a.G;
+    const int dim = is_v ? a.dv : a.d;
+    const int c0 = is_v ? 2 * a.G * a.d + (unit - 2 * a.G) * a.dv : unit * a.d;  // first channel, also the column of `in`
+    const int C = 2 * a.G * a.d + a.H * a.dv, keep = a.taps - 1;
+    float wv[EPL][TAPS], win[EPL][TAPS];  // index b: the input b rows back; win[.][0] is not kept
+    int ch[EPL];
+    bool on[EPL];
+#pragma unroll
+    for (int e = 0; e < EPL; ++e) {
+        on[e] = lane + e * 64 < dim;
+        ch[e] = c0 + (on[e] ? lane + e * 64 : 0);
+#pragma unroll
+        for (int b = 0; b < TAPS; ++b) {
+            const float w = a.w[(size_t)ch[e] * a.taps + max(keep - b, 0)];
+            wv[e][b] = b <= keep ? w : 0.f;
+        }
+    }
+    int s = seq_of_row(t0, a.seq_q_start, a.S);
+    int q0 = a.seq_q_start[s], len = a.seq_q_len[s];
+    auto load_window = [&](int t) {  // the inputs before row t
+        const float* st = a.state + (size_t)a.seq_slot[s] * keep * C;
+#pragma unroll
+        for (int e = 0; e < EPL; ++e)
+#pragma unroll
+            for (int b = 1; b < TAPS; ++b) {
+                win[e][b] = 0.f;
+                if (b > keep) continue;
+                const int idx = t - b - q0;  // counted from the request's first row; the same for the whole wave
+                win[e][b] = idx >= 0 ? sum_at(a.in, t - b, ch[e]) : st[(size_t)(keep + idx) * C + ch[e]];
+            }
+    };
+    load_window(t0);
+#pragma unroll 1
+    for (int r = 0; r < ROWS; ++r) {
+        const int t = t0 + r;
+        if (t >= a.T) return;
+        if (t >= q0 + len) {  // the next request's first row
+            do {
+                ++s;
+                q0 = a.seq_q_start[s];
+                len = a.seq_q_len[s];
+            } while (len == 0 && s + 1 < a.S);
+            load_window(t);
+        }
+        float y[EPL], ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < EPL; ++e) {
+            const float cur = sum_at(a.in, t, ch[e]);
+            float acc = wv[e][0] * cur;
+#pragma unroll
+            for (int b = 1; b < TAPS; ++b) acc += wv[e][b] * win[e][b];
+#pragma unroll
+            for (int b = TAPS - 1; b > 1; --b) win[e][b] = win[e][b - 1];
+            if constexpr (TAPS > 1) win[e][1] = cur;
+            y[e] = on[e] ? silu_f(acc) : 0.f;
+            ss += y[e] * y[e];
+        }
+        if (len == 1 && keep > 0) {
+            float* st = a.state + (size_t)a.seq_slot[s] * keep * C;
+#pragma unroll
+            for (int e = 0; e < EPL; ++e)
+                if (on[e]) {
+#pragma unroll
+                    for (int b = 1; b < TAPS; ++b)
+                        if (b <= keep) st[(size_t)(keep - b) * C + ch[e]] = win[e][b];
+                }
+        }
+        if (!is_v) {
+            ss = wave_sum(ss);
+            const float f = (unit < a.G ? a.q_scale : 1.0f) / sqrtf(ss + UNIT_EPS);
+            float* dst = (unit < a.G ? a.q + (size_t)t * a.G * a.d + unit * a.d : a.k + (size_t)t * a.G * a.d + (unit - a.G) * a.d);
+#pragma unroll
+            for (int e = 0; e < EPL; ++e)
+                if (on[e]) dst[lane + e * 64] = y[e] * f;
+        } else {
+            float* dst = a.v + (size_t)t * a.H * a.dv + (unit - 2 * a.G) * a.dv;
+#pragma unroll
+            for (int e = 0; e < EPL; ++e)
+                if (on[e]) dst[lane + e * 64] = y[e];
+        }
+    }
+}
+
+// The convolution's state after the step, for requests of several rows: their last taps - 1 inputs, old ones where the
+// step brought fewer.  Comes after the kernel above.
+__global__ __launch_bounds__(256) void delta_conv_state_kernel(Sums in, float* __restrict__ state, const int* __restrict__ seq_q_start,
+                                                               const int* __restrict__ seq_q_len, const int* __restrict__ seq_slot, int C, int taps) {
+    const int s = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+    const int n = seq_q_len[s], q0 = seq_q_start[s], keep = taps - 1;
+    if (c >= C || n <= 1) return;
+    float* st = state + (size_t)seq_slot[s] * keep * C + c;
+    float v[MAX_TAPS];
+    for (int i = 0; i < keep; ++i) {
+        const int idx = n - keep + i;  // among the step's rows; negative: an older input
+        v[i] = idx >= 0 ? sum_at(in, q0 + idx, c) : st[(size_t)(keep + idx) * C];
+    }
+    for (int i = 0; i < keep; ++i) st[(size_t)i * C] = v[i];
+}
+
+// ---- gated linear attention's decays ------------------------------------------------------------------------
+// alpha[t, c] = sigmoid(z)^(1 / tau) with z = b[c] + sum_r wt[r, c] low[t, r], low = R columns of `in` from col on; `wt` is the
+// projection transposed, [R, C].  A block takes ROWS rows and 256 channels: a weight is read once for all of its rows.
+template <int ROWS>
+__global__ __launch_bounds__(256) void key_decay_kernel(Sums in, int col, const float* __restrict__ wt, const float* __restrict__ b,
+                                                        float inv_tau, float* __restrict__ alpha, int T, int C, int R) {
+    extern __shared__ float low[];  // [ROWS][R]
+    const int t0 = blockIdx.x * ROWS, c = blockIdx.y * 256 + threadIdx.x;
+    const int nr = min(ROWS, T - t0);
+    for (int i = threadIdx.x; i < nr * R; i += 256) low[i] = sum_at(in, t0 + i / R, col + i % R);
+    __syncthreads();
+    if (c >= C) return;
+    float acc[ROWS];
+    const float bias = b[c];
+#pragma unroll
+    for (int k = 0; k < ROWS; ++k) acc[k] = bias;
+#pragma unroll 8
+    for (int r = 0; r < R; ++r) {
+        const float w = wt[(size_t)r * C + c];
+#pragma unroll
+        for (int k = 0; k < ROWS; ++k) acc[k] += w * low[(k < nr ? k : 0) * R + r];
+    }
+#pragma unroll
+    for (int k = 0; k < ROWS; ++k)
+        if (k < nr) alpha[(size_t)(t0 + k) * C + c] = expf(-inv_tau * softplus_f(-acc[k]));
+}
+
+// ---- what both rules' kernels read --------------------------------------------------------------------------
+struct StateArgs {
+    Sums q, k, v;            // columns q_col + head * d, k_col + head * d, v_col + h * dv; q and k: of head h / (H / G)
+    int q_col, k_col, v_col;
+    float q_scale;
+    const float* decay;      // gated linear: alpha [T, H * d]; delta rule: lg [T, H]
+    const float* beta;       // [T, H] (delta rule)
+    Sums gate;               // columns g_col + h * dv
+    int g_col;
+    const float* norm;       // [dv]
+    float eps;
+    float* state;            // [slots, H, d, dvp]
+    const int* seq_q_start;
+    const int* seq_q_len;
+    const int* seq_slot;
+    int S;
+    elem_t* out;             // [T, ld_out], zeros behind H * dv
+    int ld_out;
+    int T, H, G, d, dv, dvp;
+};
+
+__device__ __forceinline__ void zero_tail(const StateArgs& a, int t) {
+    for (int c = a.H * a.dv + threadIdx.x; c < a.ld_out; c += blockDim.x) a.out[(size_t)t * a.ld_out + c] = from_f32<elem_t>(0.f);
+}
+
+// ---- single rows --------------------------------------------------------------------------------------------
+// Request s has the one row s.  A thread holds 4 neighbouring value channels of every RG-th key channel; all of the state is
+// asked for at once.  Both products with the old state (S^T k and S^T q) are summed in one pass: with the state's new
+// value S' = g S + k u^T,  o = S'^T q = g S^T q + (q . k) u.
+template <int CG, int DP, bool DELTA>
+__global__ __launch_bounds__(256) void state_step_kernel(StateArgs a) {
+    constexpr int RG = 256 / CG, RPT = DP / RG, W = 4 * CG;
+    __shared__ float qs[DP], ks[DP], ws[DP], us[W];
+    __shared__ float red[DELTA ? 2 : 1][RG][W];
+    __shared__ float scratch[4];
+    const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, cg = tid % CG, rg = tid / CG;
+    const int kh = h / (a.H / a.G);
+    float* st = a.state + (((size_t)a.seq_slot[t] * a.H + h) * a.d) * a.dvp + cg * 4;
+    const bool col_in = cg * 4 < a.dvp;
+    f32x4 S[RPT];
+#pragma unroll
+    for (int j = 0; j < RPT; ++j) {
+        const int i = j * RG + rg;
+        S[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
+        if (col_in && i < a.d) S[j] = *reinterpret_cast<const f32x4*>(st + (size_t)i * a.dvp);
+    }
+    const bool live = tid < a.dv;
+    const float vc = live ? sum_at(a.v, t, a.v_col + h * a.dv + tid) : 0.f;
+    const float zc = live ? sum_at(a.gate, t, a.g_col + h * a.dv + tid) : 0.f;
+    float qk = 0.f;
+    for (int i = tid; i < DP; i += 256) {
+        const bool in = i < a.d;
+        const float qv = in ? sum_at(a.q, t, a.q_col + kh * a.d + i) * a.q_scale : 0.f, kv = in ? sum_at(a.k, t, a.k_col + kh * a.d + i) : 0.f;
+        qs[i] = qv;
+        ks[i] = kv;
+        if (!DELTA) ws[i] = in ? a.decay[((size_t)t * a.H + h) * a.d + i] : 0.f;
+        qk += qv * kv;
+    }
+    const float g = DELTA ? expf(a.decay[(size_t)t * a.H + h]) : 1.f, beta = DELTA ? a.beta[(size_t)t * a.H + h] : 1.f;
+    if (!DELTA && tid < W) us[tid] = vc;
+    if (DELTA) qk = block_sum<256>(qk, scratch);  // (a barrier: the rows are in LDS)
+    else __syncthreads();
+    {
+        f32x4 pk = (f32x4){0.f, 0.f, 0.f, 0.f}, pq = pk;
+        const f32x4 u4 = DELTA ? pk : *reinterpret_cast<const f32x4*>(&us[cg * 4]);
+#pragma unroll
+        for (int j = 0; j < RPT; ++j) {
+            const int i = j * RG + rg;
+            const float kv = ks[i], qv = qs[i];
+            if (DELTA) pk += S[j] * kv;
+            else S[j] = S[j] * ws[i] + u4 * kv;
+            pq += S[j] * qv;
+        }
+        *reinterpret_cast<f32x4*>(&red[0][rg][cg * 4]) = pq;
+        if constexpr (DELTA) *reinterpret_cast<f32x4*>(&red[1][rg][cg * 4]) = pk;
+    }
+    __syncthreads();
+    float o = 0.f;
+    if (tid < W) {
+        float sk = 0.f;
+#pragma unroll
+        for (int r = 0; r < RG; ++r) {
+            o += red[0][r][tid];
+            if constexpr (DELTA) sk += red[1][r][tid];
+        }
+        if constexpr (DELTA) {
+            const float u = beta * (vc - g * sk);
+            us[tid] = u;
+            o = g * o + qk * u;
+        }
+    }
+    const float ss = block_sum<256>(live ? o * o : 0.f, scratch);
+    if constexpr (DELTA) {  // (block_sum's barriers: the writes are in LDS)
+        const f32x4 u4 = *reinterpret_cast<const f32x4*>(&us[cg * 4]);
+#pragma unroll
+        for (int j = 0; j < RPT; ++j) S[j] = S[j] * g + u4 * ks[j * RG + rg];
+    }
+#pragma unroll
+    for (int j = 0; j < RPT; ++j) {
+        const int i = j * RG + rg;
+        if (col_in && i < a.d) *reinterpret_cast<f32x4*>(st + (size_t)i * a.dvp) = S[j];
+    }
+    if (live) a.out[(size_t)t * a.ld_out + h * a.dv + tid] = from_f32<elem_t>(o / sqrtf(ss / (float)a.dv + a.eps) * a.norm[tid] * silu_f(zc));
+    if (h == 0) zero_tail(a, t);
+}
+
+// ---- gated linear attention over many rows ---------------------------------------------------------------------
+// A thread is a value channel and holds its column of S in registers (DP of them; the rows beyond d stay zero).  Tokens come
+// WALK_BATCH at a time through LDS; the next batch's numbers are asked for before the current batch is walked.  seg_len 0: a
+// block walks all of a request's rows.  Else a request's rows are cut into segments (numbered by piece_of): LOCAL walks
+// each from zero and leaves what it adds (carry [numbers, H, d, dvp]) and the product of its decays (cdec [numbers, H, d]),
+// the carry kernel replaces what it adds by the state that comes into it, and the second walk makes the outputs.
+constexpr int WALK_BATCH = 8;
+struct WalkArgs {
+    StateArgs a;
+    int seg_len;
+    float* carry;
+    float* cdec;
+};
+
+template <int DP, int NT, bool LOCAL>
+__global__ __launch_bounds__(NT) void state_walk_kernel(WalkArgs w) {
+    constexpr int TB = WALK_BATCH, NW = NT / 64, KPT = TB * DP / NT;
+    const StateArgs& a = w.a;
+    __shared__ __align__(16) float qs[LOCAL ? 1 : TB][DP], ks[TB][DP], ws[TB][DP];
+    __shared__ float vs[TB][NT], os[LOCAL ? 1 : TB][NT], part[TB][NW];
+    const int h = blockIdx.y, j = threadIdx.x, d = a.d;
+    Piece pc{(int)blockIdx.x, 0};
+    if (w.seg_len) pc = piece_of(blockIdx.x, w.seg_len, a.seq_q_start, a.S);
+    const int left = a.seq_q_len[pc.s] - pc.first;
+    if (left <= 0) return;  // the same for the whole block
+    const int n = w.seg_len ? min(left, w.seg_len) : left;
+    const bool last = n == left;
+    if (LOCAL && last) return;  // nobody needs what the last segment passes on
+    const int q0 = a.seq_q_start[pc.s] + pc.first, kh = h / (a.H / a.G);
+    const bool live = j < a.dv;
+    const size_t head = (size_t)d * a.dvp;
+    float* st = a.state + ((size_t)a.seq_slot[pc.s] * a.H + h) * head + j;
+    float* pass = w.seg_len ? w.carry + ((size_t)blockIdx.x * a.H + h) * head + j : nullptr;
+    float S[DP];
+    {
+        const float* from = w.seg_len ? pass : st;
+#pragma unroll
+        for (int i = 0; i < DP; ++i) S[i] = (!LOCAL && live && i < d) ? from[(size_t)i * a.dvp] : 0.f;
+    }
+    float pq[LOCAL ? 1 : KPT], pk[KPT], pw[KPT], pv[TB], pg[LOCAL ? 1 : TB];
+    const float nw = live ? a.norm[j] : 0.f;
+    auto fetch = [&](int j0) {  // tokens j0 .. j0 + TB - 1 (the last one again beyond the end)
+#pragma unroll
+        for (int u = 0; u < KPT; ++u) {
+            const int idx = j + u * NT, b = idx / DP, c = idx % DP;
+            const int t = q0 + min(j0 + b, n - 1), cc = min(c, d - 1);
+            pk[u] = sum_at(a.k, t, a.k_col + kh * d + cc);
+            pw[u] = a.decay[((size_t)t * a.H + h) * d + cc];
+            if (!LOCAL) pq[u] = sum_at(a.q, t, a.q_col + kh * d + cc);
+        }
+#pragma unroll
+        for (int b = 0; b < TB; ++b) {
+            const int t = q0 + min(j0 + b, n - 1), c = h * a.dv + (live ? j : 0);
+            pv[b] = sum_at(a.v, t, a.v_col + c);
+            if (!LOCAL) pg[b] = sum_at(a.gate, t, a.g_col + c);
+        }
+    };
+    float prod[LOCAL ? (DP + NT - 1) / NT : 1];  // LOCAL: the product of the decays of key channels j, j + NT, ...
+#pragma unroll
+    for (int u = 0; u < (LOCAL ? (DP + NT - 1) / NT : 1); ++u) prod[u] = 1.f;
+    fetch(0);
+    for (int j0 = 0; j0 < n; j0 += TB) {
+        const int nb = min(TB, n - j0);
+        __syncthreads();  // the batch before has been walked by everyone
+#pragma unroll
+        for (int u = 0; u < KPT; ++u) {
+            const int idx = j + u * NT, b = idx / DP, c = idx % DP;
+            const bool in = c < d;
+            ks[b][c] = in ? pk[u] : 0.f;
+            ws[b][c] = in ? pw[u] : 0.f;
+            if (!LOCAL) qs[b][c] = in ? pq[u] * a.q_scale : 0.f;
+        }
+        float gv[LOCAL ? 1 : TB];
+#pragma unroll
+        for (int b = 0; b < TB; ++b) {
+            vs[b][j] = live ? pv[b] : 0.f;
+            if (!LOCAL) gv[b] = pg[b];
+        }
+        __syncthreads();
+        if (j0 + TB < n) fetch(j0 + TB);
+        if constexpr (LOCAL) {
+#pragma unroll
+            for (int u = 0; u < (DP + NT - 1) / NT; ++u) {
+                const int c = j + u * NT;
+                if (c < DP)
+                    for (int b = 0; b < nb; ++b) prod[u] *= ws[b][c];
+            }
+        }
+        // the batch's outputs wait in LDS, each in its thread's own place: their norms are worked out together behind the walk
+#pragma unroll 1
+        for (int b = 0; b < nb; ++b) {
+            const float vj = vs[b][j];
+            float o0 = 0.f, o1 = 0.f, o2 = 0.f, o3 = 0.f;  // four chains of sums side by side
+#pragma unroll
+            for (int i = 0; i < DP; i += 4) {
+                const float4 k4 = *reinterpret_cast<const float4*>(&ks[b][i]);
+                const float4 w4 = *reinterpret_cast<const float4*>(&ws[b][i]);
+                S[i] = fmaf(w4.x, S[i], k4.x * vj);
+                S[i + 1] = fmaf(w4.y, S[i + 1], k4.y * vj);
+                S[i + 2] = fmaf(w4.z, S[i + 2], k4.z * vj);
+                S[i + 3] = fmaf(w4.w, S[i + 3], k4.w * vj);
+                if (!LOCAL) {
+                    const float4 q4 = *reinterpret_cast<const float4*>(&qs[b][i]);
+                    o0 = fmaf(q4.x, S[i], o0);
+                    o1 = fmaf(q4.y, S[i + 1], o1);
+                    o2 = fmaf(q4.z, S[i + 2], o2);
+                    o3 = fmaf(q4.w, S[i + 3], o3);
+                }
+            }
+            if (!LOCAL) os[b][j] = (o0 + o1) + (o2 + o3);
+        }
+        if constexpr (!LOCAL) {
+            float ob[TB], ss[TB];
+#pragma unroll
+            for (int b = 0; b < TB; ++b) {
+                ob[b] = (live && b < nb) ? os[b][j] : 0.f;
+                ss[b] = wave_sum(ob[b] * ob[b]);
+            }
+            if constexpr (NW > 1) {  // the head's other waves
+                if ((j & 63) == 0) {
+#pragma unroll
+                    for (int b = 0; b < TB; ++b) part[b][j >> 6] = ss[b];
+                }
+                __syncthreads();
+#pragma unroll
+                for (int b = 0; b < TB; ++b) {
+                    ss[b] = part[b][0];
+#pragma unroll
+                    for (int q = 1; q < NW; ++q) ss[b] += part[b][q];
+                }
+            }
+#pragma unroll
+            for (int b = 0; b < TB; ++b) {
+                const int t = q0 + j0 + b;
+                if (b >= nb) continue;
+                if (live) a.out[(size_t)t * a.ld_out + h * a.dv + j] = from_f32<elem_t>(ob[b] / sqrtf(ss[b] / (float)a.dv + a.eps) * nw * silu_f(gv[b]));
+                if (h == 0) zero_tail(a, t);
+            }
+        }
+    }
+    if (LOCAL) {
+#pragma unroll
+        for (int u = 0; u < (LOCAL ? (DP + NT - 1) / NT : 1); ++u)
+            if (j + u * NT < d) w.cdec[((size_t)blockIdx.x * a.H + h) * d + j + u * NT] = prod[u];
+    }
+    if (j >= a.dvp) return;  // the columns that fill dv up hold zeros
+    if (LOCAL) {
+#pragma unroll
+        for (int i = 0; i < DP; ++i)
+            if (i < d) pass[(size_t)i * a.dvp] = S[i];
+    } else if (last) {
+#pragma unroll
+        for (int i = 0; i < DP; ++i)
+            if (i < d) st[(size_t)i * a.dvp] = S[i];
+    }
+}
+
+// Between the two walks: S_in(next) = diag(product of the segment's decays) S_in + what the segment adds, from the slot's state.
+__global__ __launch_bounds__(256) void state_carry_kernel(WalkArgs w) {
+    const StateArgs& a = w.a;
+    const int s = blockIdx.x, h = blockIdx.y, idx = blockIdx.z * 256 + threadIdx.x, head = a.d * a.dvp;
+    if (idx >= head) return;
+    const int i = idx / a.dvp, base = piece_base(s, w.seg_len, a.seq_q_start);
+    const int nseg = (a.seq_q_len[s] + w.seg_len - 1) / w.seg_len;
+    float Sin = a.state[((size_t)a.seq_slot[s] * a.H + h) * head + idx];
+    for (int seg = 0; seg < nseg; ++seg) {
+        const size_t at = (size_t)(base + seg) * a.H + h;
+        float* p = w.carry + at * head + idx;
+        const bool more = seg + 1 < nseg;
+        const float dec = more ? w.cdec[at * a.d + i] : 0.f, add = more ? *p : 0.f;
+        *p = Sin;
+        Sin = dec * Sin + add;
+    }
+}
+
+// ---- the delta rule over many rows: chunks of 64 tokens -----------------------------------------------------------
+// For the tokens i, j = 0 .. n - 1 of a chunk, L_i = sum of lg up to i (so exp(L_i - L_j) is the decay from j to i), and the
+// state S before the chunk, unrolling the rule gives
+//     (I + A) U = diag(beta) V - diag(beta e^L) K S,     A_ij = beta_i exp(L_i - L_j) (k_i . k_j)  for j < i, else 0
+//     o_i = e^(L_i) S^T q_i + sum_{j <= i} exp(L_i - L_j) (q_i . k_j) u_j
+//     S after = e^(L_n) S + sum_j exp(L_n - L_j) k_j u_j^T.
+// delta_solve (all chunks side by side): W = (I + A)^-1 diag(beta e^L) K and U0 = (I + A)^-1 diag(beta) V by forward
+// substitution in blocks of 16 tokens; delta_pass (a request's chunks in order): U = U0 - W S, the state before every chunk and
+// the state after the last; delta_out (all chunks side by side): o, its norm and gate.  All products run on the matrix
+// cores' 32-bit form.  The order of sums within a chunk does not depend on where the portion was cut other than through
+// the chunk's own start.
+constexpr int CH = 64;        // tokens of a chunk: one a lane where their decays are summed
+constexpr int SL = 64;        // channels of q and k that a block holds in LDS at a time
+constexpr int LDP = SL + 4;   // their row stride
+
+struct DeltaChunkArgs {
+    StateArgs a;   // q and k already unit vectors and scaled: one partial sum, columns from 0
+    float* W;      // [T, H, dk16]
+    float* U0;     // [T, H, dv]
+    float* U;      // [T, H, dv]
+    float* Sb;     // [numbers, H, dk16, dv16]: the state before each chunk
+    int dk16, dv16;
+};
+
+__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// lane i: the sum of lg of the chunk's tokens up to i (tokens beyond n add nothing)
+__device__ __forceinline__ float decay_sums(const float* __restrict__ lg, int t0, int n, int H, int h, int lane) {
+    float v = lane < n ? lg[(size_t)(t0 + lane) * H + h] : 0.f;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+        const float up = __shfl_up(v, o, WAVE);
+        if (lane >= o) v += up;
+    }
+    return v;
+}
+
+// CH rows of channels c0 .. c0 + SL of `src` (row stride ld) into LDS, zeros beyond n rows and d channels
+__device__ __forceinline__ void load_slice(float* dst, const float* __restrict__ src, size_t ld, int c0, int n, int d) {
+    for (int idx = threadIdx.x; idx < CH * SL; idx += 256) {
+        const int r = idx / SL, c = idx % SL;
+        dst[r * LDP + c] = (r < n && c0 + c < d) ? src[r * ld + c0 + c] : 0.f;
+    }
+}
+
+// The lower triangle's ten tiles of 16 x 16 over four waves: tile number -> row and column tile.
+__device__ __forceinline__ void lower_tile(int t, int& rt, int& ct) {
+    rt = t >= 6 ? 3 : t >= 3 ? 2 : t >= 1 ? 1 : 0;
+    ct = t - (rt * (rt + 1)) / 2;
+}
+
+__global__ __launch_bounds__(256) void delta_solve_kernel(DeltaChunkArgs p) {
+    const StateArgs& a = p.a;
+    __shared__ __align__(16) float Ks[CH * LDP], As[CH * LDP];
+    __shared__ float Ls[CH], bs[CH];
+    const Piece pc = piece_of(blockIdx.x, CH, a.seq_q_start, a.S);
+    const int left = a.seq_q_len[pc.s] - pc.first;
+    if (left <= 0) return;  // the same for the whole block
+    const int n = min(left, CH), t0 = a.seq_q_start[pc.s] + pc.first, h = blockIdx.y, kh = h / (a.H / a.G);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
+    const size_t ldk = (size_t)a.G * a.d;
+    const float* kp = a.k.p + (size_t)t0 * ldk + (size_t)kh * a.d;
+    if (wave == 0) {
+        Ls[lane] = decay_sums(a.decay, t0, n, a.H, h, lane);
+        bs[lane] = lane < n ? a.beta[(size_t)(t0 + lane) * a.H + h] : 0.f;
+    }
+    const int used = (n + 15) / 16, tiles = used * (used + 1) / 2;  // row tiles with tokens, and their lower triangle
+    f32x4 acc[3];
+#pragma unroll
+    for (int u = 0; u < 3; ++u) acc[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < a.d; c0 += SL) {
+        if (c0) __syncthreads();
+        load_slice(Ks, kp, ldk, c0, n, a.d);
+        __syncthreads();
+#pragma unroll
+        for (int u = 0; u < 3; ++u) {
+            const int tile = wave + u * 4;
+            if (tile >= tiles) continue;
+            int rt, ct;
+            lower_tile(tile, rt, ct);
+#pragma unroll
+            for (int kk = 0; kk < SL / 16; ++kk) {
+                const f32x4 x = *reinterpret_cast<const f32x4*>(&Ks[(rt * 16 + r16) * LDP + kk * 16 + grp * 4]);
+                const f32x4 y = *reinterpret_cast<const f32x4*>(&Ks[(ct * 16 + r16) * LDP + kk * 16 + grp * 4]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[u] = mfma_f32(x[i], y[i], acc[u]);
+            }
+        }
+    }
+#pragma unroll
+    for (int u = 0; u < 3; ++u) {
+        const int tile = wave + u * 4;
+        if (tile >= tiles) continue;
+        int rt, ct;
+        lower_tile(tile, rt, ct);
+        const int j = ct * 16 + r16;
+#pragma unroll
+        for (int ii = 0; ii < 4; ++ii) {
+            const int i = rt * 16 + grp * 4 + ii;
+            As[i * LDP + j] = j < i ? bs[i] * expf(Ls[i] - Ls[j]) * acc[u][ii] : 0.f;
+        }
+    }
+    __syncthreads();
+    // the diagonal's blocks are replaced by the inverses of I + A there: a wave a block, a lane a column
+    if (wave < used && lane < 16) {
+        float* D = As + wave * 16 * LDP + wave * 16;
+        float x[16];
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            float v = i == lane ? 1.f : 0.f;
+#pragma unroll
+            for (int j = 0; j < i; ++j) v = fmaf(-D[i * LDP + j], x[j], v);
+            x[i] = v;
+        }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) D[i * LDP + lane] = x[i];
+    }
+    __syncthreads();
+    // Right sides, 16 columns a wave at a time: K's (filled up to dk16 with zeros), then V's.  A block of 16 solved rows is an
+    // accumulator, which serves the blocks below as an operand as it is (see delta_pass_kernel).
+    const size_t ldv = (size_t)a.H * a.dv;
+    for (int ct = wave; ct < (p.dk16 + p.dv16) / 16; ct += 4) {
+        const bool is_k = ct * 16 < p.dk16;
+        const int c = is_k ? ct * 16 + r16 : ct * 16 - p.dk16 + r16;
+        const bool in = c < (is_k ? a.d : a.dv);
+        const float* src = is_k ? kp + (in ? c : 0) : a.v.p + (size_t)t0 * ldv + (size_t)h * a.dv + (in ? c : 0);
+        const size_t ld = is_k ? ldk : ldv;
+        f32x4 X[4];
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int r = b * 16 + grp * 4 + i;
+                const float v = src[(size_t)min(r, n - 1) * ld];
+                X[b][i] = in ? v * (bs[r] * (is_k ? expf(Ls[r]) : 1.f)) : 0.f;  // (beta is zero beyond the chunk's end)
+            }
+#pragma unroll
+        for (int b = 0; b < 4; ++b) {
+            if (b >= used) continue;
+            f32x4 R = X[b];
+#pragma unroll
+            for (int e = 0; e < b; ++e) {
+                const f32x4 m = *reinterpret_cast<const f32x4*>(&As[(b * 16 + r16) * LDP + e * 16 + grp * 4]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) R = mfma_f32(-m[i], X[e][i], R);
+            }
+            const f32x4 m = *reinterpret_cast<const f32x4*>(&As[(b * 16 + r16) * LDP + b * 16 + grp * 4]);
+            f32x4 Y = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int i = 0; i < 4; ++i) Y = mfma_f32(m[i], R[i], Y);
+            X[b] = Y;
+        }
+        float* dst = is_k ? p.W + ((size_t)t0 * a.H + h) * p.dk16 + c : p.U0 + (size_t)t0 * ldv + (size_t)h * a.dv + c;
+        const size_t ldw = is_k ? (size_t)a.H * p.dk16 : ldv;
+#pragma unroll
+        for (int b = 0; b < 4; ++b)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int r = b * 16 + grp * 4 + i;
+                if (r < n && (is_k || in)) dst[(size_t)r * ldw] = X[b][i];
+            }
+    }
+}
+
+// A block walks a request's chunks for one head and 16 value channels.  Wave w holds the state's rows of the 16-wide tiles
+// w * KT .. w * KT + KT - 1 as accumulators, which serve as operands as they are: lane (grp, r16) holds rows grp * 4 + i of
+// column r16, and supplies them as the four steps i of a product over those rows.
+template <int KT>
+__global__ __launch_bounds__(256) void delta_pass_kernel(DeltaChunkArgs p) {
+    const StateArgs& a = p.a;
+    __shared__ f32x4 part[2][4][4][64];
+    const int s = blockIdx.z, h = blockIdx.y, n0 = blockIdx.x * 16, kh = h / (a.H / a.G);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
+    const int q0 = a.seq_q_start[s], len = a.seq_q_len[s];
+    if (len <= 0) return;
+    const int col = n0 + r16;
+    const bool col_in = col < a.dv;
+    float* st = a.state + ((size_t)a.seq_slot[s] * a.H + h) * a.d * a.dvp;
+    const int base = piece_base(s, CH, a.seq_q_start);
+    f32x4 S[KT];
+    int k0[KT];
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+        k0[kt] = (wave * KT + kt) * 16;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int k = k0[kt] + grp * 4 + i;
+            S[kt][i] = (k < a.d && col_in) ? st[(size_t)k * a.dvp + col] : 0.f;
+        }
+    }
+    f32x4 Wf[4][KT], Kf[KT][4], Uf[4];
+    float lsum = 0.f;
+    const size_t ldk = (size_t)a.G * a.d, ldu = (size_t)a.H * a.dv;
+    auto fetch = [&](int ch) {  // a chunk's operands; rows beyond its end and channels beyond the head are zeros
+        const int t0 = q0 + ch * CH, n = min(CH, len - ch * CH);
+        lsum = decay_sums(a.decay, t0, n, a.H, h, lane);
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            const int r = rt * 16 + r16;
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt) {
+                Wf[rt][kt] = (f32x4){0.f, 0.f, 0.f, 0.f};
+                if (r < n && k0[kt] < p.dk16)
+                    Wf[rt][kt] = *reinterpret_cast<const f32x4*>(p.W + ((size_t)(t0 + r) * a.H + h) * p.dk16 + k0[kt] + grp * 4);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int j = rt * 16 + grp * 4 + i;
+                const bool row = j < n;
+                Uf[rt][i] = (row && col_in) ? p.U0[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] : 0.f;
+#pragma unroll
+                for (int kt = 0; kt < KT; ++kt) {
+                    const int k = k0[kt] + r16;
+                    Kf[kt][rt][i] = (row && k < a.d) ? a.k.p[(size_t)(t0 + j) * ldk + (size_t)kh * a.d + k] : 0.f;
+                }
+            }
+        }
+    };
+    const int nch = (len + CH - 1) / CH;
+    fetch(0);
+    for (int ch = 0; ch < nch; ++ch) {
+        const int t0 = q0 + ch * CH, n = min(CH, len - ch * CH), buf = ch & 1;
+        // the state before the chunk, for the kernel that makes the outputs
+        float* sb = p.Sb + ((size_t)(base + ch) * a.H + h) * p.dk16 * p.dv16 + col;
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt)
+            if (k0[kt] < p.dk16) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) sb[(size_t)(k0[kt] + grp * 4 + i) * p.dv16] = S[kt][i];
+            }
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            f32x4 ws = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) ws = mfma_f32(Wf[rt][kt][i], S[kt][i], ws);
+            part[buf][wave][rt][lane] = ws;
+        }
+        const float l = lsum, total = __shfl(l, 63, WAVE), gall = expf(total), e = expf(total - l);
+        f32x4 Us[4], Kc[KT][4];
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            Us[rt] = Uf[rt];
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt) Kc[kt][rt] = Kf[kt][rt];
+        }
+        __syncthreads();  // the waves' shares of W S are in LDS (the other half was read before they were written)
+        if (ch + 1 < nch) fetch(ch + 1);
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            f32x4 ws = part[buf][0][rt][lane];
+#pragma unroll
+            for (int w = 1; w < 4; ++w) ws += part[buf][w][rt][lane];
+            Us[rt] -= ws;
+            if (rt == wave && col_in) {
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int j = rt * 16 + grp * 4 + i;
+                    if (j < n) p.U[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] = Us[rt][i];
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i) Us[rt][i] *= __shfl(e, rt * 16 + grp * 4 + i, WAVE);
+        }
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) {
+            S[kt] *= gall;
+#pragma unroll
+            for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) S[kt] = mfma_f32(Kc[kt][rt][i], Us[rt][i], S[kt]);
+        }
+    }
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int k = k0[kt] + grp * 4 + i;
+            if (k < a.d && col_in) st[(size_t)k * a.dvp + col] = S[kt][i];
+        }
+}
+
+// Wave w makes the value channels of the 16-wide tiles w, w + 4, ... (CT of them) for all of a chunk's tokens.
+template <int CT>
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
+    const StateArgs& a = p.a;
+    __shared__ __align__(16) float Qs[CH * LDP], Ks[CH * LDP];
+    __shared__ float Ls[CH], rows[4][CH];
+    const Piece pc = piece_of(blockIdx.x, CH, a.seq_q_start, a.S);
+    const int left = a.seq_q_len[pc.s] - pc.first;
+    if (left <= 0) return;  // the same for the whole block
+    const int n = min(left, CH), t0 = a.seq_q_start[pc.s] + pc.first, h = blockIdx.y, kh = h / (a.H / a.G);
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
+    const int used = (n + 15) / 16, tiles = used * (used + 1) / 2;
+    const size_t ldk = (size_t)a.G * a.d, ldu = (size_t)a.H * a.dv;
+    const float* qp = a.q.p + (size_t)t0 * ldk + (size_t)kh * a.d;
+    const float* kp = a.k.p + (size_t)t0 * ldk + (size_t)kh * a.d;
+    const float* sb = p.Sb + ((size_t)blockIdx.x * a.H + h) * p.dk16 * p.dv16;
+    if (wave == 0) Ls[lane] = decay_sums(a.decay, t0, n, a.H, h, lane);
+    f32x4 O[4][CT], P[3];
+#pragma unroll
+    for (int u = 0; u < 3; ++u) P[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) O[rt][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < a.d; c0 += SL) {
+        f32x4 B[SL / 16][CT];  // the state's rows c0 .. c0 + SL of this wave's columns
+#pragma unroll
+        for (int kk = 0; kk < SL / 16; ++kk)
+#pragma unroll
+            for (int c = 0; c < CT; ++c) {
+                const int col = (wave + 4 * c) * 16 + r16;
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int k = c0 + kk * 16 + grp * 4 + i;
+                    B[kk][c][i] = (k < p.dk16 && col < p.dv16) ? sb[(size_t)k * p.dv16 + col] : 0.f;
+                }
+            }
+        if (c0) __syncthreads();
+        load_slice(Qs, qp, ldk, c0, n, a.d);
+        load_slice(Ks, kp, ldk, c0, n, a.d);
+        __syncthreads();
+#pragma unroll
+        for (int u = 0; u < 3; ++u) {
+            const int tile = wave + u * 4;
+            if (tile >= tiles) continue;
+            int rt, ct;
+            lower_tile(tile, rt, ct);
+#pragma unroll
+            for (int kk = 0; kk < SL / 16; ++kk) {
+                const f32x4 x = *reinterpret_cast<const f32x4*>(&Qs[(rt * 16 + r16) * LDP + kk * 16 + grp * 4]);
+                const f32x4 y = *reinterpret_cast<const f32x4*>(&Ks[(ct * 16 + r16) * LDP + kk * 16 + grp * 4]);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) P[u] = mfma_f32(x[i], y[i], P[u]);
+            }
+        }
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            if (rt >= used) continue;
+#pragma unroll
+            for (int kk = 0; kk < SL / 16; ++kk) {
+                const f32x4 x = *reinterpret_cast<const f32x4*>(&Qs[(rt * 16 + r16) * LDP + kk * 16 + grp * 4]);
+#pragma unroll
+                for (int c = 0; c < CT; ++c)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) O[rt][c] = mfma_f32(x[i], B[kk][c][i], O[rt][c]);
+            }
+        }
+    }
+    __syncthreads();  // everyone has read the keys: the scores take their place
+    float* Ps = Ks;
+#pragma unroll
+    for (int u = 0; u < 3; ++u) {
+        const int tile = wave + u * 4;
+        if (tile >= tiles) continue;
+        int rt, ct;
+        lower_tile(tile, rt, ct);
+        const int j = ct * 16 + r16;
+#pragma unroll
+        for (int ii = 0; ii < 4; ++ii) {
+            const int i = rt * 16 + grp * 4 + ii;
+            Ps[i * LDP + j] = j <= i ? expf(Ls[i] - Ls[j]) * P[u][ii] : 0.f;
+        }
+    }
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int ii = 0; ii < 4; ++ii) {
+            const float f = expf(Ls[rt * 16 + grp * 4 + ii]);
+#pragma unroll
+            for (int c = 0; c < CT; ++c) O[rt][c][ii] *= f;
+        }
+    f32x4 Uf[4][CT];
+#pragma unroll
+    for (int jt = 0; jt < 4; ++jt)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) {
+            const int col = (wave + 4 * c) * 16 + r16;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int j = jt * 16 + grp * 4 + i;
+                Uf[jt][c][i] = (j < n && col < a.dv) ? p.U[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] : 0.f;
+            }
+        }
+    __syncthreads();
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) {
+        if (rt >= used) continue;
+#pragma unroll
+        for (int jt = 0; jt <= rt; ++jt) {
+            const f32x4 x = *reinterpret_cast<const f32x4*>(&Ps[(rt * 16 + r16) * LDP + jt * 16 + grp * 4]);
+#pragma unroll
+            for (int c = 0; c < CT; ++c)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) O[rt][c] = mfma_f32(x[i], Uf[jt][c][i], O[rt][c]);
+        }
+    }
+    // the heads' norms: a row's squares over this wave's columns, then over the waves
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int ii = 0; ii < 4; ++ii) {
+            float ss = 0.f;
+#pragma unroll
+            for (int c = 0; c < CT; ++c) ss += O[rt][c][ii] * O[rt][c][ii];  // columns beyond dv are zeros
+#pragma unroll
+            for (int o = 1; o < 16; o <<= 1) ss += __shfl_xor(ss, o, WAVE);
+            if (r16 == 0) rows[wave][rt * 16 + grp * 4 + ii] = ss;
+        }
+    __syncthreads();
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int ii = 0; ii < 4; ++ii) {
+            const int i = rt * 16 + grp * 4 + ii, t = t0 + i;
+            if (i >= n) continue;
+            const float ss = (rows[0][i] + rows[1][i]) + (rows[2][i] + rows[3][i]);
+            const float inv = 1.0f / sqrtf(ss / (float)a.dv + a.eps);
+#pragma unroll
+            for (int c = 0; c < CT; ++c) {
+                const int col = (wave + 4 * c) * 16 + r16;
+                if (col < a.dv)
+                    a.out[(size_t)t * a.ld_out + h * a.dv + col] =
+                        from_f32<elem_t>(O[rt][c][ii] * inv * a.norm[col] * silu_f(sum_at(a.gate, t, a.g_col + h * a.dv + col)));
+            }
+        }
+    if (h == 0)
+        for (int i = 0; i < n; ++i) zero_tail(a, t0 + i);
+}
+
+}  // namespace ms
+
+using namespace ms;
+
+extern "C" int ms_gated_state_max_taps() { return MAX_TAPS; }
+extern "C" int ms_gated_state_max_dim() { return MAX_DIM; }
+extern "C" int ms_gated_state_max_rank() { return 1536; }  // eight rows of it lie in LDS
+extern "C" int ms_delta_chunk() { return CH; }
+
+// in: float [n_partials, T, ld].  many: requests of several rows may be among the step's (their states are then brought up
+// to date by a second launch).
+extern "C" int ms_delta_rows(const float* in, int n_partials, int ld, const float* w, float* state, const float* a_log, const float* dt_bias,
+                             const int* seq_q_start, const int* seq_q_len, const int* seq_slot, int S, float* q, float* k, float* v,
+                             float* beta, float* lg, int T, int H, int G, int d, int dv, int taps, int b_col, int a_col, float q_scale,
+                             int many, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && S > 0 && n_partials > 0 && H > 0 && G > 0 && H % G == 0, "delta rows: T=%d S=%d, %d heads over %d", T, S, H, G);
+    MS_REQUIRE(d > 0 && d <= MAX_DIM && dv > 0 && dv <= MAX_DIM, "delta rows: heads of %d and %d, at most %d", d, dv, MAX_DIM);
+    MS_REQUIRE(taps >= 1 && taps <= MAX_TAPS && (taps == 1 || state), "delta rows: %d taps (1 to %d) and their state", taps, MAX_TAPS);
+    const int C = 2 * G * d + H * dv;
+    MS_REQUIRE(ld >= C && b_col >= 0 && a_col >= 0 && b_col + H <= ld && a_col + H <= ld, "delta rows: rows of %d numbers", ld);
+    MS_REQUIRE(in && w && a_log && dt_bias && seq_q_start && seq_q_len && seq_slot && q && k && v && beta && lg, "delta rows: a buffer is missing");
+    const DeltaRowsArgs a{Sums{in, n_partials, (size_t)T * ld, ld}, w, state, a_log, dt_bias, seq_q_start, seq_q_len, seq_slot, S,
+                          q, k, v, beta, lg, T, H, G, d, dv, taps, b_col, a_col, q_scale};
+    const int units = 2 * G + H + 1, wide = d > dv ? d : dv;
+#define MS_ROWS(TP, E, R) hipLaunchKernelGGL((delta_rows_kernel<TP, E, R>), dim3(ceil_div(T, R), ceil_div(units, 4)), dim3(256), 0, stream, a)
+#define MS_ROWS_E(TP, R)                     \
+    do {                                     \
+        if (wide <= 64) MS_ROWS(TP, 1, R);   \
+        else if (wide <= 128) MS_ROWS(TP, 2, R); \
+        else MS_ROWS(TP, 4, R);              \
+    } while (0)
+    const bool tall = T >= 256;
+    if (taps <= 4) {
+        if (tall) MS_ROWS_E(4, 8);
+        else MS_ROWS_E(4, 1);
+    } else {
+        if (tall) MS_ROWS_E(MAX_TAPS, 8);
+        else MS_ROWS_E(MAX_TAPS, 1);
+    }
+#undef MS_ROWS_E
+#undef MS_ROWS
+    if (int rc = check_launch("delta rows")) return rc;
+    if (taps == 1 || !many) return 0;
+    hipLaunchKernelGGL(delta_conv_state_kernel, dim3(S, ceil_div(C, 256)), dim3(256), 0, stream, a.in, state, seq_q_start, seq_q_len, seq_slot, C, taps);
+    return check_launch("delta rows, convolution state");
+}
+
+extern "C" int ms_key_decay(const float* in, int n_partials, int ld, int col, const float* wt, const float* b, float tau, float* alpha, int T,
+                            int C, int R, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && C > 0 && R > 0 && n_partials > 0 && col >= 0 && col + R <= ld, "key decay: T=%d C=%d, %d columns at %d of %d", T, C, R, col, ld);
+    MS_REQUIRE(R <= ms_gated_state_max_rank(), "key decay: a bottleneck of %d, at most %d", R, ms_gated_state_max_rank());
+    MS_REQUIRE(tau > 0.f && in && wt && b && alpha, "key decay: tau %g, or a buffer is missing", (double)tau);
+    const Sums rows{in, n_partials, (size_t)T * ld, ld};
+    if (T >= 128)
+        hipLaunchKernelGGL(key_decay_kernel<8>, dim3(ceil_div(T, 8), ceil_div(C, 256)), dim3(256), (size_t)8 * R * sizeof(float), stream, rows, col,
+                           wt, b, 1.0f / tau, alpha, T, C, R);
+    else
+        hipLaunchKernelGGL(key_decay_kernel<1>, dim3(T, ceil_div(C, 256)), dim3(256), (size_t)R * sizeof(float), stream, rows, col, wt, b, 1.0f / tau,
+                           alpha, T, C, R);
+    return check_launch("key decay");
+}
+
+static int check_state(const StateArgs& a, const char* what) {
+    MS_REQUIRE(a.T > 0 && a.S > 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.H <= 65535, "%s: T=%d S=%d, %d heads over %d", what, a.T, a.S, a.H, a.G);
+    MS_REQUIRE(a.d > 0 && a.d <= MAX_DIM && a.dv > 0 && a.dv <= MAX_DIM, "%s: heads of %d and %d, at most %d", what, a.d, a.dv, MAX_DIM);
+    MS_REQUIRE(a.dvp >= a.dv && a.dvp % 4 == 0 && a.dvp < a.dv + 4 && a.ld_out >= a.H * a.dv, "%s: values of %d in %d, rows of %d", what, a.dv, a.dvp, a.ld_out);
+    MS_REQUIRE(a.q_col >= 0 && a.q_col + a.G * a.d <= a.q.ld && a.k_col >= 0 && a.k_col + a.G * a.d <= a.k.ld && a.v_col >= 0 &&
+                   a.v_col + a.H * a.dv <= a.v.ld && a.g_col >= 0 && a.g_col + a.H * a.dv <= a.gate.ld,
+               "%s: columns beyond the rows", what);
+    MS_REQUIRE(a.q.p && a.k.p && a.v.p && a.gate.p && a.decay && a.norm && a.state && a.seq_q_start && a.seq_q_len && a.seq_slot && a.out,
+               "%s: a buffer is missing", what);
+    MS_REQUIRE((reinterpret_cast<uintptr_t>(a.state)) % 16 == 0, "%s: the state must be 16-byte aligned", what);
+    return 0;
+}
+
+template <bool DELTA>
+static int launch_step(const StateArgs& a, hipStream_t stream) {
+    MS_REQUIRE(a.S == a.T, "single rows: %d rows of %d requests", a.T, a.S);
+    const dim3 grid(a.T, a.H);
+#define MS_STEP(CG, DP) hipLaunchKernelGGL((state_step_kernel<CG, DP, DELTA>), grid, dim3(256), 0, stream, a)
+#define MS_STEP_D(CG)                    \
+    do {                                 \
+        if (a.d <= 32) MS_STEP(CG, 32);  \
+        else if (a.d <= 64) MS_STEP(CG, 64); \
+        else if (a.d <= 128) MS_STEP(CG, 128); \
+        else MS_STEP(CG, 256);           \
+    } while (0)
+    if (a.dv <= 32) MS_STEP_D(8);
+    else if (a.dv <= 64) MS_STEP_D(16);
+    else if (a.dv <= 128) MS_STEP_D(32);
+    else MS_STEP_D(64);
+#undef MS_STEP_D
+#undef MS_STEP
+    return check_launch("gated state, single rows");
+}
+
+// Gated linear attention.  rows: float [n_partials, T, ld] with q [H, d], k [H, d], v [H, dv] and gate [H, dv] at their columns;
+// alpha float [T, H * d].  single: every request has one row.  seg_len > 0: segments side by side with carry float
+// [T / seg_len + S, H, d, dvp] and cdec float [T / seg_len + S, H, d] as workspace.
+extern "C" int ms_gated_linear(const float* rows, int n_partials, int ld, int q_col, int k_col, int v_col, int g_col, float q_scale,
+                               const float* alpha, const float* norm, float eps, float* state, const int* seq_q_start, const int* seq_q_len,
+                               const int* seq_slot, int S, void* out, int ld_out, int T, int H, int d, int dv, int dvp, int single,
+                               int seg_len, float* carry, float* cdec, hipStream_t stream) {
+    const Sums in{rows, n_partials, (size_t)T * ld, ld};
+    const StateArgs a{in, in, in, q_col, k_col, v_col, q_scale, alpha, nullptr, in, g_col, norm, eps, state, seq_q_start, seq_q_len, seq_slot, S,
+                      (elem_t*)out, ld_out, T, H, H, d, dv, dvp};
+    MS_REQUIRE(n_partials > 0, "gated linear: no rows");
+    if (int rc = check_state(a, "gated linear")) return rc;
+    if (single) return launch_step<false>(a, stream);
+    MS_REQUIRE(seg_len == 0 || (seg_len > 0 && carry && cdec), "gated linear: segments of %d need their workspace", seg_len);
+    const WalkArgs w{a, seg_len, carry, cdec};
+#define MS_WALK(DP, NT, LOCAL, X) hipLaunchKernelGGL((state_walk_kernel<DP, NT, LOCAL>), dim3(X, H), dim3(NT), 0, stream, w)
+#define MS_WALK_N(DP, LOCAL, X)                   \
+    do {                                          \
+        if (dv <= 64) MS_WALK(DP, 64, LOCAL, X);  \
+        else if (dv <= 128) MS_WALK(DP, 128, LOCAL, X); \
+        else MS_WALK(DP, 256, LOCAL, X);          \
+    } while (0)
+#define MS_WALK_D(LOCAL, X)                       \
+    do {                                          \
+        if (d <= 32) MS_WALK_N(32, LOCAL, X);     \
+        else if (d <= 64) MS_WALK_N(64, LOCAL, X); \
+        else if (d <= 128) MS_WALK_N(128, LOCAL, X); \
+        else MS_WALK_N(256, LOCAL, X);            \
+    } while (0)
+    if (seg_len == 0) {
+        MS_WALK_D(false, S);
+        return check_launch("gated linear");
+    }
+    const int numbers = T / seg_len + S;
+    MS_WALK_D(true, numbers);
+    if (int rc = check_launch("gated linear, segments from zero")) return rc;
+    hipLaunchKernelGGL(state_carry_kernel, dim3(S, H, ceil_div(d * dvp, 256)), dim3(256), 0, stream, w);
+    if (int rc = check_launch("gated linear, states between segments")) return rc;
+    MS_WALK_D(false, numbers);
+#undef MS_WALK_D
+#undef MS_WALK_N
+#undef MS_WALK
+    return check_launch("gated linear, segments");
+}
+
+// The gated delta rule.  q, k float [T, G * d] (unit vectors, q scaled), v float [T, H * dv], lg and beta float [T, H] as
+// ms_delta_rows leaves them; gate: columns g_col on of float [n_partials, T, ld].  single: every request has one row; else
+// W float [T, H, dk16], U0 and U float [T, H, dv] and Sb float [T / 64 + S, H, dk16, dv16] are the workspace.
+extern "C" int ms_gated_delta(const float* q, const float* k, const float* v, const float* lg, const float* beta, const float* gate,
+                              int n_partials, int ld, int g_col, const float* norm, float eps, float* state, const int* seq_q_start,
+                              const int* seq_q_len, const int* seq_slot, int S, void* out, int ld_out, int T, int H, int G, int d, int dv,
+                              int dvp, int single, float* W, float* U0, float* U, float* Sb, hipStream_t stream) {
+    const Sums qs{q, 1, 0, G * d}, ks{k, 1, 0, G * d}, vs{v, 1, 0, H * dv}, gs{gate, n_partials, (size_t)T * ld, ld};
+    const StateArgs a{qs, ks, vs, 0, 0, 0, 1.0f, lg, beta, gs, g_col, norm, eps, state, seq_q_start, seq_q_len, seq_slot, S,
+                      (elem_t*)out, ld_out, T, H, G, d, dv, dvp};
+    MS_REQUIRE(n_partials > 0 && beta, "gated delta: no rows");
+    if (int rc = check_state(a, "gated delta")) return rc;
+    if (single) return launch_step<true>(a, stream);
+    MS_REQUIRE(W && U0 && U && Sb && S <= 65535, "gated delta: chunks of %d need their workspace", CH);
+    MS_REQUIRE((reinterpret_cast<uintptr_t>(W)) % 16 == 0, "gated delta: the workspace must be 16-byte aligned");
+    const DeltaChunkArgs p{a, W, U0, U, Sb, ceil_div(d, 16) * 16, ceil_div(dv, 16) * 16};
+    const int numbers = T / CH + S;
+    hipLaunchKernelGGL(delta_solve_kernel, dim3(numbers, H), dim3(256), 0, stream, p);
+    if (int rc = check_launch("gated delta, chunks solved")) return rc;
+    const dim3 grid(ceil_div(dv, 16), H, S);
+    if (d <= 64) hipLaunchKernelGGL(delta_pass_kernel<1>, grid, dim3(256), 0, stream, p);
+    else if (d <= 128) hipLaunchKernelGGL(delta_pass_kernel<2>, grid, dim3(256), 0, stream, p);
+    else hipLaunchKernelGGL(delta_pass_kernel<4>, grid, dim3(256), 0, stream, p);
+    if (int rc = check_launch("gated delta, states between chunks")) return rc;
+    if (dv <= 64) hipLaunchKernelGGL(delta_out_kernel<1>, dim3(numbers, H), dim3(256), 0, stream, p);
+    else if (dv <= 128) hipLaunchKernelGGL(delta_out_kernel<2>, dim3(numbers, H), dim3(256), 0, stream, p);
+    else hipLaunchKernelGGL(delta_out_kernel<4>, dim3(numbers, H), dim3(256), 0, stream, p);
+    return check_launch("gated delta, outputs");
+}

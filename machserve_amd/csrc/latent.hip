@@ -85,11 +85,10 @@ __global__ __launch_bounds__(256) void latent_row_kernel(LatentRowArgs a) {
         krow[c] = v;
         vcol[(size_t)c * a.ps] = v;
     }
-    const float pos = (float)a.positions[t];
     const float* kr = row + a.q_rank + a.rank;
     for (int i = threadIdx.x; i < a.rot / 2; i += 256) {
         float sn, cs;
-        sincosf(pos * a.inv_freq[i], &sn, &cs);
+        angle_cos_sin(a.positions[t], a.inv_freq[i], cs, sn);
         sn *= a.cs_factor;
         cs *= a.cs_factor;
         const int iu = a.halves ? i : 2 * i, iv = a.halves ? i + a.rot / 2 : 2 * i + 1;
@@ -106,7 +105,6 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const float* __restri
                                                            elem_t* __restrict__ plain, elem_t* __restrict__ att, int H, int d, int dp,
                                                            int rot, int rank, int hd, int halves) {
     const int t = blockIdx.x;
-    const float pos = (float)positions[t];
     const float* qr = q + (size_t)t * H * (d + rot);
     for (int c = threadIdx.x; c < H * dp; c += 256) {
         const int h = c / dp, e = c - h * dp;
@@ -119,7 +117,7 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const float* __restri
         elem_t* dst = att + ((size_t)t * H + h) * hd + rank;
         if (i < half) {
             float sn, cs;
-            sincosf(pos * inv_freq[i], &sn, &cs);
+            angle_cos_sin(positions[t], inv_freq[i], cs, sn);
             sn *= cs_factor;
             cs *= cs_factor;
             const int iu = halves ? i : 2 * i, iv = halves ? i + half : 2 * i + 1;

@@ -11,23 +11,11 @@
 // depends on its own request alone.  Short steps walk a request's rows token after token; long portions are walked in
 // segments side by side whose incoming states a carry kernel chains, so that cuts of a prompt differ by that chain's
 // 32-bit rounding and by nothing else.
-#include "common.cuh"
+#include "recurrence.cuh"
 #include <type_traits>
 
 namespace ms {
 
-__device__ __forceinline__ int seq_of_row(int t, const int* __restrict__ seq_q_start, int S) {
-    int lo = 0, hi = S - 1;
-    while (lo < hi) {
-        const int mid = (lo + hi + 1) >> 1;
-        if (seq_q_start[mid] <= t) lo = mid;
-        else hi = mid - 1;
-    }
-    return lo;
-}
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 __device__ __forceinline__ float gelu_tanh_f(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
 
 constexpr int MAX_TAPS = 16;

@@ -11,24 +11,9 @@
 // tokens were cut into steps by rounding only, and never on what else the step holds.  Decays, step sizes,
 // exponentials, the states and all sums are 32-bit in every build; the element type stores the projections'
 // outputs and is the operand type of lightning attention's products.
-#include "common.cuh"
+#include "recurrence.cuh"
 
 namespace ms {
-
-// The request that row t belongs to: the last s with seq_q_start[s] <= t (starts ascend with s).
-__device__ __forceinline__ int seq_of_row(int t, const int* __restrict__ seq_q_start, int S) {
-    int lo = 0, hi = S - 1;
-    while (lo < hi) {
-        const int mid = (lo + hi + 1) >> 1;
-        if (seq_q_start[mid] <= t) lo = mid;
-        else hi = mid - 1;
-    }
-    return lo;
-}
-
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 
 // ---- causal convolution per channel --------------------------------------------------
 // out[t, c] = silu(b[c] + sum_k w[c, k] * in[t - (taps - 1 - k), c]); an input before the step's first row of the

@@ -8,14 +8,11 @@
 // the tokens' B, C, step sizes and decays come through LDS a few tokens at a time, so every thread reads them as
 // broadcasts, four states at once.  Long portions are cut into segments that are walked side by side (see the kernel).
 // Everything is 32-bit in every build.
-#include "common.cuh"
+#include "recurrence.cuh"
 
 namespace ms {
 
 constexpr int SSD_TOK = 8;  // tokens whose B, C, dt and decay a block holds in LDS at a time
-
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 struct SsdArgs {
     const float* xbc;      // [T, ld_xbc]: x [H, P], B [G, N], C [G, N] before their SiLU

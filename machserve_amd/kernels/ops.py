@@ -1027,6 +1027,26 @@ class HipOps:
         self._check(self._core, self._core.ms_pair_norm_add(_ptr(x), _ptr(pa), _c_int(pa.shape[0]), _ptr(wa), _ptr(pb), _c_int(pb.shape[0]),
                                                             _ptr(wb), _ptr(weight), _c_int(T), _c_int(d), _c_float(eps), self._stream()))
 
+    def norm_add_weighted(self, x: torch.Tensor, pa: torch.Tensor, fa: float, pb: torch.Tensor, fb: float, weight: torch.Tensor, eps: float) -> None:
+        """``x += rmsnorm(fa sum(pa) + fb sum(pb)) * weight``: two branches side by side, each given as the float32 partial sums
+        ``[P, T, d]`` of its last product."""
+        T, d = x.shape
+        self._want(x, torch.float32, "norm_add_weighted stream")
+        for p in (pa, pb):
+            self._want(p, torch.float32, "norm_add_weighted sums", p.shape[0], T, d)
+        self._want(weight, torch.float32, "norm_add_weighted weight", d)
+        self._check(self._core, self._core.ms_norm_add_weighted(_ptr(x), _ptr(pa), _c_int(pa.shape[0]), _c_float(fa), _ptr(pb), _c_int(pb.shape[0]),
+                                                                _c_float(fb), _ptr(weight), _c_int(T), _c_int(d), _c_float(eps), self._stream()))
+
+    def open_pass(self, x: torch.Tensor, first: Optional[torch.Tensor], row: torch.Tensor) -> None:
+        """``x += first + row`` in place: the rows of ``first`` (None: nothing) and one row for all, in 32-bit."""
+        T, d = x.shape
+        self._want(x, torch.float32, "open_pass stream")
+        if first is not None:
+            self._want(first, torch.float32, "open_pass rows", T, d)
+        self._want(row, torch.float32, "open_pass row", d)
+        self._check(self._core, self._core.ms_open_pass(_ptr(x), _ptr(first), _ptr(row), _c_int(T), _c_int(d), self._stream()))
+
     def gate_mul(self, sums: torch.Tensor, activation: str) -> torch.Tensor:
         """``act(sums[:, :n]) * sums[:, n:]`` in the element type for float32 ``sums [T, 2 n]``: the gated product of a
         feed-forward whose gate and up projections carry biases."""
@@ -1470,6 +1490,125 @@ class HipOps:
         z = _c_void(proj.data_ptr() + z_col * 4)
         self._check(lib, lib.ms_gated_group_norm(_ptr(y), z, _c_int(proj.shape[1]), _ptr(weight), _ptr(out), _c_int(out_cols), _c_int(T),
                                                  _c_int(n), _c_int(groups), _c_float(eps), self._stream()))
+        return out
+
+    # ------------------------------------------------------------------ matrix-valued states under gates
+    def gated_state_limits(self) -> dict:
+        lib = self._extra_lib("gated_state")
+        return {"taps": lib.ms_gated_state_max_taps(), "dim": lib.ms_gated_state_max_dim(), "rank": lib.ms_gated_state_max_rank()}
+
+    def _state_operands(self, what, sums, norm_w, state, H, d, dv, seqs):
+        if sums.dim() == 2:
+            sums = sums.unsqueeze(0)
+        self._want(sums, torch.float32, f"{what} rows")
+        self._want(norm_w, torch.float32, f"{what} norm weight", dv)
+        dvp = -(-dv // 4) * 4
+        self._want(state, torch.float32, f"{what} state", state.shape[0], H, d, dvp)
+        S = self._seq_operands(what, *seqs)
+        return sums, dvp, S
+
+    def key_decay(self, sums: torch.Tensor, col: int, w_t: torch.Tensor, bias: torch.Tensor, tau: float) -> torch.Tensor:
+        """Decays of gated linear attention, float32 ``[T, C]``: ``sigmoid(z)^(1 / tau)`` with ``z = low @ w_t + bias``, ``low`` being
+        columns ``col .. col + R`` of the float32 partial sums ``[P, T, N]`` and ``w_t [R, C]`` the second projection, transposed."""
+        lib = self._extra_lib("gated_state")
+        if sums.dim() == 2:
+            sums = sums.unsqueeze(0)
+        P, T, N = sums.shape
+        R, C = w_t.shape
+        self._want(sums, torch.float32, "key decay rows")
+        self._want(w_t, torch.float32, "key decay weight (transposed)")
+        self._want(bias, torch.float32, "key decay bias", C)
+        alpha = torch.empty((T, C), dtype=torch.float32, device=sums.device)
+        self._check(lib, lib.ms_key_decay(_ptr(sums), _c_int(P), _c_int(N), _c_int(col), _ptr(w_t), _ptr(bias), _c_float(tau), _ptr(alpha),
+                                          _c_int(T), _c_int(C), _c_int(R), self._stream()))
+        return alpha
+
+    STATE_SEGMENT = 32  # rows of a segment of gated linear attention
+
+    def gated_linear(self, sums: torch.Tensor, alpha: torch.Tensor, norm_w: torch.Tensor, eps: float, q_scale: float, state: torch.Tensor,
+                     seq_q_start: torch.Tensor, seq_q_len: torch.Tensor, seq_slot: torch.Tensor, H: int, d: int, dv: int, out_cols: int,
+                     single: bool = False) -> torch.Tensor:
+        """Gated linear attention over the step's rows.  ``sums`` float32 ``[P, T, N]``: q ``[H, d]``, k ``[H, d]``, v ``[H, dv]``, gate
+        ``[H, dv]``, then anything; ``alpha`` float32 ``[T, H d]``; per head from ``state [slots, H, d, dv up to a multiple of 4]``:
+        ``S <- diag(alpha) S + k v^T``, ``o = S^T (q_scale q)``.  Returns ``o / rms(o) * norm_w * silu(gate)`` (the root mean square over a
+        head's ``dv``) ``[T, out_cols]`` in the element type, zeros behind ``H dv``.  ``single``: every request has one row."""
+        lib = self._extra_lib("gated_state")
+        sums, dvp, S = self._state_operands("gated linear", sums, norm_w, state, H, d, dv, (seq_q_start, seq_q_len, seq_slot))
+        P, T, N = sums.shape
+        self._want(alpha, torch.float32, "gated linear decays", T, H * d)
+        if single and S != T:
+            raise KernelError(f"gated linear: {T} rows of {S} requests are not single rows")
+        out = torch.empty((T, out_cols), dtype=self.dtype, device=sums.device)
+        seg = n = 0
+        carry = cdec = None
+        if not single:
+            seg, n = self._walk_segments(T, 1, self.STATE_SEGMENT, H * d * dvp) if T // S >= self.SCAN_CHUNK_MIN_ROWS // 2 else (0, 0)
+        if seg:
+            n = T // seg + S
+            carry = torch.empty((n, H, d, dvp), dtype=torch.float32, device=sums.device)
+            cdec = torch.empty((n, H, d), dtype=torch.float32, device=sums.device)
+        self._check(lib, lib.ms_gated_linear(
+            _ptr(sums), _c_int(P), _c_int(N), _c_int(0), _c_int(H * d), _c_int(2 * H * d), _c_int(2 * H * d + H * dv), _c_float(q_scale), _ptr(alpha),
+            _ptr(norm_w), _c_float(eps), _ptr(state), _ptr(seq_q_start), _ptr(seq_q_len), _ptr(seq_slot), _c_int(S), _ptr(out), _c_int(out_cols),
+            _c_int(T), _c_int(H), _c_int(d), _c_int(dv), _c_int(dvp), _c_int(int(single)), _c_int(seg), _ptr(carry), _ptr(cdec), self._stream()))
+        return out
+
+    def delta_rows(self, sums: torch.Tensor, conv_w: torch.Tensor, conv_state: Optional[torch.Tensor], a_log: torch.Tensor, dt_bias: torch.Tensor,
+                   q_scale: float, seq_q_start: torch.Tensor, seq_q_len: torch.Tensor, seq_slot: torch.Tensor, H: int, G: int, d: int, dv: int,
+                   single: bool = False):
+        """Rows of the gated delta rule from float32 partial sums ``[P, T, N]``: q ``[G, d]``, k ``[G, d]``, v ``[H, dv]``, gate ``[H, dv]``, b ``[H]``,
+        a ``[H]``.  q, k and v pass a causal convolution (``conv_w [2 G d + H dv, taps]``, earlier inputs from ``conv_state [slots, taps - 1,
+        channels]``, which is brought up to date) and SiLU; q and k of a head become unit vectors (``x / sqrt(sum x^2 + 1e-6)``), q times
+        ``q_scale``.  Returns float32 ``(q, k [T, G d], v [T, H dv], beta = sigmoid(b), lg = -exp(a_log) softplus(a + dt_bias) [T, H])``."""
+        lib = self._extra_lib("gated_state")
+        if sums.dim() == 2:
+            sums = sums.unsqueeze(0)
+        P, T, N = sums.shape
+        C, taps = 2 * G * d + H * dv, conv_w.shape[1]
+        self._want(sums, torch.float32, "delta rows")
+        if N < C + H * dv + 2 * H:
+            raise KernelError(f"delta rows: {N} columns for {C + H * dv + 2 * H} numbers")
+        self._want(conv_w, torch.float32, "delta convolution weight", C, taps)
+        if taps > 1:
+            self._want(conv_state, torch.float32, "delta convolution state", conv_state.shape[0], taps - 1, C)
+        else:
+            conv_state = None
+        for t, name in ((a_log, "A_log"), (dt_bias, "dt_bias")):
+            self._want(t, torch.float32, f"delta {name}", H)
+        S = self._seq_operands("delta rows", seq_q_start, seq_q_len, seq_slot)
+        new = lambda n: torch.empty((T, n), dtype=torch.float32, device=sums.device)
+        q, k, v, beta, lg = new(G * d), new(G * d), new(H * dv), new(H), new(H)
+        self._check(lib, lib.ms_delta_rows(
+            _ptr(sums), _c_int(P), _c_int(N), _ptr(conv_w), _ptr(conv_state), _ptr(a_log), _ptr(dt_bias), _ptr(seq_q_start), _ptr(seq_q_len),
+            _ptr(seq_slot), _c_int(S), _ptr(q), _ptr(k), _ptr(v), _ptr(beta), _ptr(lg), _c_int(T), _c_int(H), _c_int(G), _c_int(d), _c_int(dv),
+            _c_int(taps), _c_int(C + H * dv), _c_int(C + H * dv + H), _c_float(q_scale), _c_int(int(not single)), self._stream()))
+        return q, k, v, beta, lg
+
+    def gated_delta(self, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta: torch.Tensor, lg: torch.Tensor, sums: torch.Tensor, gate_col: int,
+                    norm_w: torch.Tensor, eps: float, state: torch.Tensor, seq_q_start: torch.Tensor, seq_q_len: torch.Tensor,
+                    seq_slot: torch.Tensor, H: int, G: int, d: int, dv: int, out_cols: int, single: bool = False) -> torch.Tensor:
+        """The gated delta rule over rows as :meth:`delta_rows` leaves them, per head from ``state [slots, H, d, dv up to a multiple of
+        4]``: ``S <- exp(lg) S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``, ``o = S^T q`` (q and k of head ``h // (H / G)``).  Returns ``o /
+        rms(o) * norm_w * silu(gate)`` ``[T, out_cols]`` in the element type, zeros behind ``H dv``; the gate is columns ``gate_col`` on of
+        the float32 partial sums ``[P, T, N]``.  ``single``: every request has one row, else its rows run in chunks of 64."""
+        lib = self._extra_lib("gated_state")
+        sums, dvp, S = self._state_operands("gated delta", sums, norm_w, state, H, d, dv, (seq_q_start, seq_q_len, seq_slot))
+        P, T, N = sums.shape
+        for t, n, name in ((q, G * d, "q"), (k, G * d, "k"), (v, H * dv, "v"), (beta, H, "beta"), (lg, H, "decay")):
+            self._want(t, torch.float32, f"gated delta {name}", T, n)
+        if single and S != T:
+            raise KernelError(f"gated delta: {T} rows of {S} requests are not single rows")
+        out = torch.empty((T, out_cols), dtype=self.dtype, device=q.device)
+        W = U0 = U = Sb = None
+        if not single:
+            dk16, dv16 = -(-d // 16) * 16, -(-dv // 16) * 16
+            new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=q.device)
+            W, U0, U = new(T, H, dk16), new(T, H, dv), new(T, H, dv)
+            Sb = new(T // lib.ms_delta_chunk() + S, H, dk16, dv16)
+        self._check(lib, lib.ms_gated_delta(
+            _ptr(q), _ptr(k), _ptr(v), _ptr(lg), _ptr(beta), _ptr(sums), _c_int(P), _c_int(N), _c_int(gate_col), _ptr(norm_w), _c_float(eps), _ptr(state),
+            _ptr(seq_q_start), _ptr(seq_q_len), _ptr(seq_slot), _c_int(S), _ptr(out), _c_int(out_cols), _c_int(T), _c_int(H), _c_int(G), _c_int(d),
+            _c_int(dv), _c_int(dvp), _c_int(int(single)), _ptr(W), _ptr(U0), _ptr(U), _ptr(Sb), self._stream()))
         return out
 
     # ------------------------------------------------------------------ sampling

@@ -134,6 +134,12 @@ class ResidualStream:
         for (a, w), g in branches:
             self.ops.norm_add(self.x, self.ops.linear_split(a, w), g / float(len(branches)), eps)
 
+    def add_weighted(self, branches) -> None:
+        """``x += sum_i f_i (a_i @ w_i.T)`` for branches side by side, each given as ``((a, w), f)``."""
+        self.open()
+        for (a, w), f in branches:
+            self.x += self.ops.linear_split(a, w).sum(0) * float(f)
+
     def add(self, y: torch.Tensor) -> None:
         """``x += y`` for a part that computes its output by other means."""
         self.open()

@@ -75,6 +75,7 @@ class _Branch:
         self.bias = None
         self.tensor = None
         self.branches = None
+        self.weighted = None
         self.scaled = None
 
     def add_linear(self, a, w, bias=None) -> None:
@@ -82,6 +83,9 @@ class _Branch:
 
     def add_normed_mean(self, branches, eps) -> None:
         self.branches = (list(branches), eps)
+
+    def add_weighted(self, branches) -> None:
+        self.weighted = list(branches)
 
     def add(self, y) -> None:
         self.tensor = y
@@ -184,7 +188,9 @@ class SandwichBlock(Block):
         out = _Branch(self.rt.ops)
         part.forward(PreNormBlock._input(pre, part, stream), out, ctx)
         stream.flush()  # a norm left pending has added what was pending by now; nothing else may be
-        if out.product is not None:
+        if out.weighted is not None:
+            post.add_normed_weighted(stream, out.weighted)
+        elif out.product is not None:
             post.add_normed(stream, *out.product)
         else:
             post.add_normed_tensor(stream, out.tensor)
@@ -222,6 +228,8 @@ class PostNormBlock(Block):
         part.forward(stream.value() if getattr(part, "reads_stream", False) else stream.rows(), out, ctx)
         if out.branches is not None:
             post.add_normed_mean(stream, *out.branches)
+        elif out.weighted is not None:
+            post.add_normed_weighted(stream, out.weighted)
         elif out.product is not None:
             post.add_normed(stream, *out.product, bias=out.bias)
         else:

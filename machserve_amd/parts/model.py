@@ -91,6 +91,20 @@ class Head(Part):
         return logits
 
 
+class LoopSteps(Part):
+    """What is added to the stream ahead of each pass over looped layers: the embedding's output again (in every pass but the
+    first) and the pass's own row of a small table, both in 32-bit."""
+
+    def tensor_decls(self):
+        return [TensorDecl("step", (len(self.spec.starts), self.spec.width), "vector")]
+
+    def load(self, t):
+        self.rows = [t["step"][i].contiguous() for i in range(len(self.spec.starts))]
+
+    def open(self, number: int, stream: ResidualStream, first: Optional[torch.Tensor]) -> None:
+        self.rt.ops.open_pass(stream.open(), first if number > 0 else None, self.rows[number])
+
+
 class DecoderModel:
     def __init__(self, spec: ModelSpec, rt: Runtime):
         spec.validate()
@@ -101,6 +115,9 @@ class DecoderModel:
         for layer in spec.layers:  # a block builds its own parts from the fields of its layer's spec
             self.blocks.append(BLOCKS.get(layer.block)(layer, rt))
         self.order = list(spec.order)
+        steps = getattr(spec, "loop_steps", None)
+        self.loop_steps = LoopSteps(steps, rt) if steps is not None else None
+        self._passes = {p: t for t, p in enumerate(steps.starts)} if steps is not None else {}
         self.final_norm = NORMS.build(spec.final_norm, rt)
         self.head = HEADS.build(spec.head, rt, self.embedding)
         self._bindings, self._rebind = [], False
@@ -116,6 +133,8 @@ class DecoderModel:
             for p in b.parts():
                 out.append(p)
                 out.extend(getattr(p, "sub_parts", lambda: [])())
+        if self.loop_steps is not None:
+            out.append(self.loop_steps)
         out += [self.final_norm, self.head]
         return out
 
@@ -187,7 +206,10 @@ class DecoderModel:
         watch = self.observer
         if watch is not None:
             watch("embedding", stream.value())
+        first = x.clone() if len(self._passes) > 1 else None  # the layers add to x in place
         for p, i in enumerate(self.order):
+            if p in self._passes:
+                self.loop_steps.open(self._passes[p], stream, first)
             if self._rebind and self._bindings[p] is not None:
                 self.blocks[i].bind_cache(self._bindings[p])
             self.blocks[i].forward(stream, ctx)

@@ -62,6 +62,16 @@ class RMSNorm(Norm):
         ops = stream.ops
         ops.pair_norm_add(stream.x, ops.linear_split(a, w_a), wa, ops.linear_split(b, w_b), wb, self.weight, self.spec.eps)
 
+    def add_normed_weighted(self, stream, branches) -> None:
+        """``x += rmsnorm(fa (a @ w_a.T) + fb (b @ w_b.T)) * weight`` for two branches side by side, given as ``branches = [((a, w_a),
+        fa), ((b, w_b), fb)]`` with each branch the operands of its last product."""
+        if len(branches) != 2:
+            raise ValueError(f"{len(branches)} branches side by side under a norm: the kernel takes two")
+        ((a, w_a), fa), ((b, w_b), fb) = branches
+        stream.open()
+        ops = stream.ops
+        ops.norm_add_weighted(stream.x, ops.linear_split(a, w_a), float(fa), ops.linear_split(b, w_b), float(fb), self.weight, self.spec.eps)
+
     def normalise_sum(self, stream, alpha: float, sums, bias=None) -> None:
         """``x <- rmsnorm(alpha x + sum(sums) (+ bias)) * weight``: the norm behind a residual sum.  ``sums`` float32 ``[P, T,
         width]`` are what a branch's last product left; one kernel adds them up, normalises the row and leaves it in

@@ -1,5 +1,5 @@
 """Several mixers side by side: all read the same input, each one's output is RMS-normed over the model's width with a
-weight of its own, and the result is their mean.  The branches are mixers of any registered kind; each keeps the cache
+weight of its own, and the result is their mean; or, with factors in the spec, the sum of their outputs times those, without norms.  The branches are mixers of any registered kind; each keeps the cache
 or state it asks for, and what the branches ask for is handed on as one flat list.  A branch must end in a product
 (``add_linear``): the norms read its 32-bit sums."""
 from __future__ import annotations
@@ -32,6 +32,8 @@ class SideBySide(Mixer):
         self.branches = [MIXERS.build(b, rt) for b in spec.branches]
         if any(getattr(b, "reads_stream", False) for b in self.branches):
             raise ValueError("side_by_side: a branch that reads the 32-bit stream itself")
+        if spec.factors is not None and len(spec.factors) != len(spec.branches):
+            raise ValueError(f"side_by_side: {len(spec.factors)} factors for {len(spec.branches)} branches")
         self.norms = None
 
     @property
@@ -46,9 +48,13 @@ class SideBySide(Mixer):
         return out
 
     def tensor_decls(self):
+        if self.spec.factors is not None:
+            return []
         return [TensorDecl(f"norm.{i}", (self.spec.hidden,), "vector") for i in range(len(self.branches))]
 
     def load(self, t):
+        if self.spec.factors is not None:
+            return
         self.norms = [t[f"norm.{i}"] for i in range(len(self.branches))]
 
     # ------------------------------------------------------------------ caches: every branch's own, as one flat list
@@ -91,4 +97,7 @@ class SideBySide(Mixer):
             last = _Last()
             b.forward(h, last, ctx)
             lasts.append(last.product)
+        if self.spec.factors is not None:
+            stream.add_weighted(list(zip(lasts, self.spec.factors)))
+            return
         stream.add_normed_mean(list(zip(lasts, self.norms)), self.spec.norm_eps)

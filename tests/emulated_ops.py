@@ -321,6 +321,15 @@ class EmulatedOps:
         rms = lambda y: y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps))
         x += rms(0.5 * (rms(pa.sum(0)) * wa + rms(pb.sum(0)) * wb)) * weight
 
+    def norm_add_weighted(self, x, pa, fa, pb, fb, weight, eps):
+        y = fa * pa.sum(0) + fb * pb.sum(0)
+        x += y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps)) * weight
+
+    def open_pass(self, x, first, row):
+        if first is not None:
+            x += first
+        x += row
+
     def gate_mul(self, sums, activation):
         n = sums.shape[1] // 2
         return self._r(_act(sums[:, :n], activation) * sums[:, n:])
@@ -578,6 +587,70 @@ class EmulatedOps:
         out = torch.zeros(T, out_cols)
         out[:, :n] = g.reshape(T, n) * weight
         return self._r(out)
+
+    # ------------------------------------------------------------------ matrix-valued states under gates
+    def gated_state_limits(self):
+        return {"taps": 16, "dim": 256, "rank": 1536}
+
+    def key_decay(self, sums, col, w_t, bias, tau):
+        low = (sums if sums.dim() == 2 else sums.sum(0))[:, col:col + w_t.shape[0]]
+        return torch.exp(-torch.nn.functional.softplus(-(low @ w_t + bias), threshold=30.0) / tau)
+
+    def _normed_gated(self, o, z, norm_w, eps, out_cols):
+        """A head's o over its root mean square, times the weight and silu(z): o, z [T, H, dv]."""
+        T, H, dv = o.shape
+        y = o * (1.0 / torch.sqrt((o * o).sum(-1, keepdim=True) / dv + eps)) * norm_w * z / (1.0 + torch.exp(-z))
+        out = torch.zeros(T, out_cols)
+        out[:, :H * dv] = y.reshape(T, H * dv)
+        return self._r(out)
+
+    def gated_linear(self, sums, alpha, norm_w, eps, q_scale, state, seq_q_start, seq_q_len, seq_slot, H, d, dv, out_cols, single=False):
+        rows = sums if sums.dim() == 2 else sums.sum(0)
+        T = rows.shape[0]
+        q, k, v, z = torch.split(rows[:, :2 * H * (d + dv)], [H * d, H * d, H * dv, H * dv], dim=1)
+        q, k, v, z, alpha = q.reshape(T, H, d) * q_scale, k.reshape(T, H, d), v.reshape(T, H, dv), z.reshape(T, H, dv), alpha.view(T, H, d)
+        o = torch.zeros(T, H, dv)
+        for q0, n, slot in zip(seq_q_start.tolist(), seq_q_len.tolist(), seq_slot.tolist()):
+            S = state[slot][..., :dv].clone()
+            for t in range(q0, q0 + n):
+                S = alpha[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+                o[t] = (S * q[t][:, :, None]).sum(1)
+            state[slot][..., :dv] = S
+        return self._normed_gated(o, z, norm_w, eps, out_cols)
+
+    def delta_rows(self, sums, conv_w, conv_state, a_log, dt_bias, q_scale, seq_q_start, seq_q_len, seq_slot, H, G, d, dv, single=False):
+        rows = sums if sums.dim() == 2 else sums.sum(0)
+        T, C, taps = rows.shape[0], 2 * G * d + H * dv, conv_w.shape[1]
+        y = torch.empty(T, C)
+        for q0, n, slot in zip(seq_q_start.tolist(), seq_q_len.tolist(), seq_slot.tolist()):
+            hist = rows[q0:q0 + n, :C]
+            if taps > 1:
+                hist = torch.cat([conv_state[slot], hist], 0)
+            y[q0:q0 + n] = sum(hist[j:j + n] * conv_w[:, j] for j in range(taps))
+            if taps > 1:
+                conv_state[slot] = hist[n:]
+        y = y / (1.0 + torch.exp(-y))
+        unit = lambda x: (x / torch.sqrt((x * x).sum(-1, keepdim=True) + 1e-6)).reshape(T, G * d)
+        b, a = rows[:, C + H * dv:C + H * dv + H], rows[:, C + H * dv + H:C + H * dv + 2 * H]
+        return (unit(y[:, :G * d].reshape(T, G, d)) * q_scale, unit(y[:, G * d:2 * G * d].reshape(T, G, d)), y[:, 2 * G * d:].contiguous(),
+                torch.sigmoid(b), -torch.exp(a_log) * torch.nn.functional.softplus(a + dt_bias, threshold=30.0))
+
+    def gated_delta(self, q, k, v, beta, lg, sums, gate_col, norm_w, eps, state, seq_q_start, seq_q_len, seq_slot, H, G, d, dv, out_cols,
+                    single=False):
+        rows = sums if sums.dim() == 2 else sums.sum(0)
+        T = rows.shape[0]
+        of = torch.arange(H) // (H // G)
+        q, k, v = q.view(T, G, d)[:, of], k.view(T, G, d)[:, of], v.view(T, H, dv)
+        o = torch.zeros(T, H, dv)
+        for q0, n, slot in zip(seq_q_start.tolist(), seq_q_len.tolist(), seq_slot.tolist()):
+            S = state[slot][..., :dv].clone()
+            for t in range(q0, q0 + n):
+                S = torch.exp(lg[t])[:, None, None] * S
+                u = beta[t][:, None] * (v[t] - (S * k[t][:, :, None]).sum(1))
+                S = S + k[t][:, :, None] * u[:, None, :]
+                o[t] = (S * q[t][:, :, None]).sum(1)
+            state[slot][..., :dv] = S
+        return self._normed_gated(o, rows[:, gate_col:gate_col + H * dv].reshape(T, H, dv), norm_w, eps, out_cols)
 
     def softcap(self, logits, scale, cap):
         v = logits * scale
