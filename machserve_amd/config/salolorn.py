@@ -218,7 +218,8 @@ class SalolornConfig:
             # a layer without feed-forward does not use its second norms, should the checkpoint have them
             unused = (f"l{i}.norm2", f"l{i}.norm2b") if ff is None else ()
             if ff is not None:
-                feed = GatedMlpSpec("gated_mlp", self.width, ff, "silu", {f"{s}.weight": f"l{i}.mlp.{s}" for s in ("gate", "up", "down")})
+                feed = GatedMlpSpec("gated_mlp", self.width, ff, "silu", {f"{s}.weight": f"l{i}.mlp.{s}" for s in ("gate", "up", "down")},
+                                    fill=True)
                 norm2, norm2b = self._norm(f"l{i}.norm2"), self._norm(f"l{i}.norm2b")
             layers.append(SandwichLayerSpec("sandwich", self._mixer_spec(m, f"l{i}.mix."), feed, self._norm(f"l{i}.norm1", unused),
                                             self._norm(f"l{i}.norm1b"), norm2, norm2b))

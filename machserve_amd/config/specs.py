@@ -413,13 +413,15 @@ class PlainMlpSpec:
 
 @dataclass(frozen=True)
 class GatedMlpSpec:
-    """``down(act(gate(x)) * up(x))``; with ``bias`` every projection has one."""
+    """``down(act(gate(x)) * up(x))``; with ``bias`` every projection has one; with ``fill`` (and no biases) an intermediate size that
+    is no multiple of 8 is filled up with zeros instead of being refused."""
     kind: str
     hidden: int
     intermediate: int
     activation: str = "silu"
     tensors: Mapping[str, str] = field(default_factory=dict)
     bias: bool = False
+    fill: bool = False
 
 
 @dataclass(frozen=True)

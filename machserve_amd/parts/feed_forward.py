@@ -23,8 +23,10 @@ class GatedMlp(FeedForward):
         super().__init__(spec, rt)
         if spec.activation not in GATE_ACTIVATIONS:
             raise ValueError(f"gated_mlp: activation {spec.activation!r} is not built (built: {', '.join(sorted(GATE_ACTIVATIONS))})")
-        require_kernel_sizes(rt, "gated_mlp", [("hidden size", spec.hidden), ("intermediate size", spec.intermediate)])
         self.bias = bool(getattr(spec, "bias", False))
+        # the joint size as the kernels see it: where the spec asks for it, filled up to a multiple of 8 by rows of zeros
+        self.joint = -(-spec.intermediate // 8) * 8 if getattr(spec, "fill", False) and not self.bias else spec.intermediate
+        require_kernel_sizes(rt, "gated_mlp", [("hidden size", spec.hidden), ("intermediate size", self.joint)])
 
     def tensor_decls(self):
         s = self.spec
@@ -42,7 +44,11 @@ class GatedMlp(FeedForward):
             self.b_gate_up = torch.cat([t["gate.bias"], t["up.bias"]]).contiguous()
             self.b_down = t["down.bias"]
         else:
-            self.w_gate_up = interleave_gate_up(t["gate.weight"], t["up.weight"])
+            fill = self.joint - self.spec.intermediate
+            pad = torch.nn.functional.pad
+            self.w_gate_up = interleave_gate_up(pad(t["gate.weight"], (0, 0, 0, fill)), pad(t["up.weight"], (0, 0, 0, fill)))
+            if fill:
+                self.w_down = pad(self.w_down, (0, fill)).contiguous()
 
     def forward(self, h, stream, ctx):
         if self.bias:
@@ -52,9 +58,9 @@ class GatedMlp(FeedForward):
             stream.add_linear(self.rt.ops.gate_mul(sums, self.spec.activation), self.w_down, self.b_down)
             return
         if isinstance(h, PendingNorm):
-            a = h.linear_swiglu(self.w_gate_up, self.spec.intermediate, self.spec.activation)
+            a = h.linear_swiglu(self.w_gate_up, self.joint, self.spec.activation)
         else:
-            a = self.rt.ops.linear_swiglu(h, self.w_gate_up, self.spec.intermediate, self.spec.activation)
+            a = self.rt.ops.linear_swiglu(h, self.w_gate_up, self.joint, self.spec.activation)
         stream.add_linear(a, self.w_down)
 
 

@@ -7,7 +7,7 @@ import os
 import torch
 
 from plain import salolorn_plain as P
-from renanex_util import relative_error, relative_errors, run_schedule, tokens_of, within  # noqa: F401  (shared runners)
+from renanex_util import relative_error, relative_errors, run_schedule, tokens_of  # noqa: F401  (shared runners)
 
 
 def latent(heads, dim, rot_dim, vdim, kv_rank, scale, base=10000.0):
@@ -127,6 +127,18 @@ def plain_logits(model_dir: str, tokens, dtype=torch.float64, weights_as=None) -
 def _is_matrix(name: str, t) -> bool:
     """What a run keeps in its element type: operands of matrix products and the embedding."""
     return t.dim() == 2 and not name.endswith((".conv", ".a2", "loop.step"))
+
+
+def within(got: torch.Tensor, want: torch.Tensor, dtype) -> bool:
+    """float32: every row within rounding of sums taken in another order (a key too many or too few, a state that is lost or a
+    pass without its row is off by 1e-2 and more).  bfloat16: rounding of activations grows through the layers, so half the
+    rows must be within 4e-2; a row whose q or k comes out of its convolution next to nothing has that rounding multiplied
+    by the unit norm: at most one row in sixty may be beyond 0.25 (logits that have nothing to do with the wanted ones are
+    off by 1.4 in every row)."""
+    e = relative_errors(got, want)
+    if dtype == torch.float32:
+        return float(e.max()) < 1e-4
+    return float(e.median()) < 4e-2 and int((e > 0.25).sum()) <= max(1, e.numel() // 60)
 
 
 def cut(rid, n, sizes):
