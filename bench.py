@@ -378,6 +378,26 @@ def livovik_configs(z):
     return livovik, melerax, qwen
 
 
+def salolorn_configs(z):
+    """(Salolorn, Melerax, Qwen2) configurations of one size.  Salolorn: the gated delta rule (as many value heads as the other
+    designs have heads, half as many for q and k) behind convolutions of four taps, latent attention (a latent of 192 beside a
+    rotated part of 64), chunked attention (chunks as long as the other designs' window) beside gated linear attention (as
+    many heads, keys half as wide as values), and the delta rule again; a dense feed-forward in every layer.  No layer runs
+    twice, so that every layer's weights come from memory as in the other designs."""
+    w, H, kv, hd = z["width"], z["heads"], z["kv"], z["hd"]
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    delta = {"type": "delta", "mixer": {"heads": H, "kv_heads": H // 2, "dim": hd, "vdim": hd, "conv": 4}, "mlp": mlp}
+    lat = {"type": "latent_attention", "mlp": mlp, "mixer": {"heads": H, "dim": hd, "rot_dim": 64, "vdim": hd, "kv_rank": 192, "scale": (hd + 64) ** -0.5,
+                                                             "rot": {"base": 10000.0, "dims": 64}}}
+    par = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": kv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": z["window"]}, "rot": {"base": 250000.0, "dims": hd}},
+        "right": {"heads": H, "dim": hd // 2, "vdim": hd, "tau": 16.0}, "left_scale": 1.2, "right_scale": 1.1}}
+    salolorn = {"architecture": "Salolorn", "vocab": DESIGN_VOCAB, "width": w, "norm": {"eps": 1e-6}, "logit_scale": 0.5,
+                "layers": [delta, lat, par, delta] * (z["layers"] // 4)}
+    melerax, _, qwen = melerax_configs(z)
+    return salolorn, melerax, qwen
+
+
 def compare_designs(args) -> int:
     """Prefill (one prompt in one step) and decode (a batch of single tokens at a context, from the captured step)
     of both designs through the step function; random weights, synthetic tokens.  One JSON line."""
@@ -399,6 +419,8 @@ def compare_designs(args) -> int:
             pairs = list(zip(("befirax", "melerax", "qwen2"), befirax_configs(z)))
         elif design == "livovik":
             pairs = list(zip(("livovik", "melerax", "qwen2"), livovik_configs(z)))
+        elif design == "salolorn":
+            pairs = list(zip(("salolorn", "melerax", "qwen2"), salolorn_configs(z)))
         else:
             pairs = list(zip((design, "qwen2"), nubodra_configs(z) if design == "nubodra" else design_configs(z)))
         for name, raw in pairs:
@@ -467,12 +489,13 @@ def main() -> int:
     ap.add_argument("--designs", action="store_true",
                     help="instead of the default run: prefill and decode throughput of Renanex layers (Mamba scan, attention whose heads "
                          "exchange scores over a window, lightning attention) beside Qwen2 layers of equal sizes, at a few sizes")
-    ap.add_argument("--design", default="renanex", choices=["renanex", "nubodra", "melerax", "befirax", "livovik"],
+    ap.add_argument("--design", default="renanex", choices=["renanex", "nubodra", "melerax", "befirax", "livovik", "salolorn"],
                     help="with --designs: which design stands beside Qwen2 (nubodra: latent attention and attention behind a convolution, "
                          "beside Qwen2 layers that see every key; befirax: state-space duality, differential and latent attention and gated "
                          "experts over two residual streams, beside Melerax and Qwen2; melerax: chunked attention beside a gated linear recurrence, time mixing "
                          "and routed experts, beside Renanex and Qwen2 layers; livovik: chunked attention with sinks and gates per head and experts "
-                         "weighed at their inputs under norms behind the sums, beside Melerax and Qwen2 layers)")
+                         "weighed at their inputs under norms behind the sums, beside Melerax and Qwen2 layers; salolorn: the gated delta rule, "
+                         "latent attention, and chunked attention beside gated linear attention, beside Melerax and Qwen2 layers)")
     ap.add_argument("--design-sizes", default="small,medium", help="with --designs: which of the sizes to run (small, medium, large)")
     ap.add_argument("--record-calls", default=None, help=argparse.SUPPRESS)  # file that receives one step's operations (the traced run)
     args = ap.parse_args()

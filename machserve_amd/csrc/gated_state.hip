@@ -85,7 +85,7 @@ __global__ __launch_bounds__(256) void delta_rows_kernel(DeltaRowsArgs a) {
     const int dim = is_v ? a.dv : a.d;
     const int c0 = is_v ? 2 * a.G * a.d + (unit - 2 * a.G) * a.dv : unit * a.d;  // first channel, also the column of `in`
     const int C = 2 * a.G * a.d + a.H * a.dv, keep = a.taps - 1;
-    float wv[EPL][TAPS], win[EPL][TAPS];  // index b: the input b rows back; win[.][0] is not kept
+    float wv[EPL][TAPS], win[EPL][TAPS] = {};  // index b: the input b rows back; win[.][0] is not kept
     int ch[EPL];
     bool on[EPL];
 #pragma unroll
@@ -102,18 +102,34 @@ __global__ __launch_bounds__(256) void delta_rows_kernel(DeltaRowsArgs a) {
     int q0 = a.seq_q_start[s], len = a.seq_q_len[s];
     auto load_window = [&](int t) {  // the inputs before row t
         const float* st = a.state + (size_t)a.seq_slot[s] * keep * C;
-#pragma unroll
-        for (int e = 0; e < EPL; ++e)
+        if (keep == 0) return;
+        // a place reads the step's rows or the state (the same for the whole wave): the address is chosen, not the load
+        for (int p = 0; p < a.in.n; ++p)
 #pragma unroll
             for (int b = 1; b < TAPS; ++b) {
-                win[e][b] = 0.f;
-                if (b > keep) continue;
-                const int idx = t - b - q0;  // counted from the request's first row; the same for the whole wave
-                win[e][b] = idx >= 0 ? sum_at(a.in, t - b, ch[e]) : st[(size_t)(keep + idx) * C + ch[e]];
+                const int back = min(b, keep), idx = t - back - q0;  // counted from the request's first row
+                const bool fresh = idx >= 0;
+                const float* src = fresh ? a.in.p + p * a.in.stride + (size_t)(t - back) * a.in.ld : st + (size_t)(keep + idx) * C;
+                const bool counts = b <= keep && (fresh || p == 0);
+#pragma unroll
+                for (int e = 0; e < EPL; ++e) {
+                    const float v = src[ch[e]];
+                    win[e][b] = (p ? win[e][b] : 0.f) + (counts ? v : 0.f);
+                }
             }
     };
+    float x[ROWS][EPL];  // the rows' own inputs, all of one partial sum's loads on one straight path
+#pragma unroll
+    for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+        for (int e = 0; e < EPL; ++e) x[r][e] = 0.f;
+    for (int p = 0; p < a.in.n; ++p)
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+#pragma unroll
+            for (int e = 0; e < EPL; ++e) x[r][e] += a.in.p[p * a.in.stride + (size_t)min(t0 + r, a.T - 1) * a.in.ld + ch[e]];
     load_window(t0);
-#pragma unroll 1
+#pragma unroll
     for (int r = 0; r < ROWS; ++r) {
         const int t = t0 + r;
         if (t >= a.T) return;
@@ -128,7 +144,7 @@ __global__ __launch_bounds__(256) void delta_rows_kernel(DeltaRowsArgs a) {
         float y[EPL], ss = 0.f;
 #pragma unroll
         for (int e = 0; e < EPL; ++e) {
-            const float cur = sum_at(a.in, t, ch[e]);
+            const float cur = x[r][e];
             float acc = wv[e][0] * cur;
 #pragma unroll
             for (int b = 1; b < TAPS; ++b) acc += wv[e][b] * win[e][b];
@@ -355,19 +371,36 @@ __global__ __launch_bounds__(NT) void state_walk_kernel(WalkArgs w) {
     float pq[LOCAL ? 1 : KPT], pk[KPT], pw[KPT], pv[TB], pg[LOCAL ? 1 : TB];
     const float nw = live ? a.norm[j] : 0.f;
     auto fetch = [&](int j0) {  // tokens j0 .. j0 + TB - 1 (the last one again beyond the end)
+        // all of one partial sum's loads go out on one straight path, then the next sum's
 #pragma unroll
         for (int u = 0; u < KPT; ++u) {
             const int idx = j + u * NT, b = idx / DP, c = idx % DP;
-            const int t = q0 + min(j0 + b, n - 1), cc = min(c, d - 1);
-            pk[u] = sum_at(a.k, t, a.k_col + kh * d + cc);
-            pw[u] = a.decay[((size_t)t * a.H + h) * d + cc];
-            if (!LOCAL) pq[u] = sum_at(a.q, t, a.q_col + kh * d + cc);
+            const int t = q0 + min(j0 + b, n - 1);
+            pw[u] = a.decay[((size_t)t * a.H + h) * d + min(c, d - 1)];
         }
+        for (int part_sum = 0; part_sum < a.k.n; ++part_sum) {
+            const size_t off = part_sum * a.k.stride;  // (q, k, v and gate are columns of the same rows)
 #pragma unroll
-        for (int b = 0; b < TB; ++b) {
-            const int t = q0 + min(j0 + b, n - 1), c = h * a.dv + (live ? j : 0);
-            pv[b] = sum_at(a.v, t, a.v_col + c);
-            if (!LOCAL) pg[b] = sum_at(a.gate, t, a.g_col + c);
+            for (int u = 0; u < KPT; ++u) {
+                const int idx = j + u * NT, b = idx / DP, c = idx % DP;
+                const size_t row = off + (size_t)(q0 + min(j0 + b, n - 1)) * a.k.ld + kh * d + min(c, d - 1);
+                const float kv = a.k.p[row + a.k_col];
+                pk[u] = part_sum ? pk[u] + kv : kv;
+                if (!LOCAL) {
+                    const float qv = a.k.p[row + a.q_col];
+                    pq[u] = part_sum ? pq[u] + qv : qv;
+                }
+            }
+#pragma unroll
+            for (int b = 0; b < TB; ++b) {
+                const size_t row = off + (size_t)(q0 + min(j0 + b, n - 1)) * a.k.ld + h * a.dv + (live ? j : 0);
+                const float vv = a.k.p[row + a.v_col];
+                pv[b] = part_sum ? pv[b] + vv : vv;
+                if (!LOCAL) {
+                    const float gv = a.k.p[row + a.g_col];
+                    pg[b] = part_sum ? pg[b] + gv : gv;
+                }
+            }
         }
     };
     float prod[LOCAL ? (DP + NT - 1) / NT : 1];  // LOCAL: the product of the decays of key channels j, j + NT, ...
@@ -503,20 +536,24 @@ constexpr int CH = 64;        // tokens of a chunk: one a lane where their decay
 constexpr int SL = 64;        // channels of q and k that a block holds in LDS at a time
 constexpr int LDP = SL + 4;   // their row stride
 
+// What the kernels hand on lies per (chunk's number, head) in whole tiles of 16, zeros beyond the chunk's tokens and the head's
+// channels, with the index that an operand's four steps run over innermost: every load of an operand is 16 bytes, without
+// conditions.
 struct DeltaChunkArgs {
     StateArgs a;   // q and k already unit vectors and scaled: one partial sum, columns from 0
-    float* W;      // [T, H, dk16]
-    float* U0;     // [T, H, dv]
-    float* U;      // [T, H, dv]
-    float* Sb;     // [numbers, H, dk16, dv16]: the state before each chunk
+    float* W;      // [numbers, H, CH, dk16]
+    float* Kt;     // [numbers, H, dk16, CH]: exp(L_n - L_j) k_j
+    float* U0;     // [numbers, H, dv16, CH]
+    float* U;      // [numbers, H, dv16, CH]
+    float* Sb;     // [numbers, H, dv16, dk16]: the state before each chunk
+    float* total;  // [numbers, H]: exp(L_n)
     int dk16, dv16;
 };
 
 __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-// lane i: the sum of lg of the chunk's tokens up to i (tokens beyond n add nothing)
-__device__ __forceinline__ float decay_sums(const float* __restrict__ lg, int t0, int n, int H, int h, int lane) {
-    float v = lane < n ? lg[(size_t)(t0 + lane) * H + h] : 0.f;
+// lane i: the sum of v over lanes 0 .. i
+__device__ __forceinline__ float lane_sums(float v, int lane) {
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
         const float up = __shfl_up(v, o, WAVE);
@@ -525,11 +562,28 @@ __device__ __forceinline__ float decay_sums(const float* __restrict__ lg, int t0
     return v;
 }
 
-// CH rows of channels c0 .. c0 + SL of `src` (row stride ld) into LDS, zeros beyond n rows and d channels
-__device__ __forceinline__ void load_slice(float* dst, const float* __restrict__ src, size_t ld, int c0, int n, int d) {
-    for (int idx = threadIdx.x; idx < CH * SL; idx += 256) {
-        const int r = idx / SL, c = idx % SL;
-        dst[r * LDP + c] = (r < n && c0 + c < d) ? src[r * ld + c0 + c] : 0.f;
+// lane i: the sum of lg of the chunk's tokens up to i (tokens beyond n add nothing)
+__device__ __forceinline__ float decay_sums(const float* __restrict__ lg, int t0, int n, int H, int h, int lane) {
+    return lane_sums(lane < n ? lg[(size_t)(t0 + lane) * H + h] : 0.f, lane);
+}
+
+// CH rows of channels c0 .. c0 + SL of `src` (row stride ld), zeros beyond n rows and d channels: asked for here, a number of
+// every fourth row a thread ...
+struct Slice {
+    float v[CH * SL / 256];
+};
+__device__ __forceinline__ void ask_slice(Slice& t, const float* __restrict__ src, size_t ld, int c0, int n, int d) {
+    const int c = min(c0 + (int)(threadIdx.x % SL), d - 1), r0 = threadIdx.x / SL;
+#pragma unroll
+    for (int u = 0; u < CH * SL / 256; ++u) t.v[u] = src[(size_t)min(r0 + u * (256 / SL), n - 1) * ld + c];
+}
+// ... and put into LDS here
+__device__ __forceinline__ void put_slice(float* dst, const Slice& t, int c0, int n, int d) {
+    const int c = threadIdx.x % SL, r0 = threadIdx.x / SL;
+#pragma unroll
+    for (int u = 0; u < CH * SL / 256; ++u) {
+        const int r = r0 + u * (256 / SL);
+        dst[r * LDP + c] = (r < n && c0 + c < d) ? t.v[u] : 0.f;
     }
 }
 
@@ -550,18 +604,46 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaChunkArgs p) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
     const size_t ldk = (size_t)a.G * a.d;
     const float* kp = a.k.p + (size_t)t0 * ldk + (size_t)kh * a.d;
+    const size_t at = (size_t)blockIdx.x * a.H + h;
     if (wave == 0) {
         Ls[lane] = decay_sums(a.decay, t0, n, a.H, h, lane);
         bs[lane] = lane < n ? a.beta[(size_t)(t0 + lane) * a.H + h] : 0.f;
     }
     const int used = (n + 15) / 16, tiles = used * (used + 1) / 2;  // row tiles with tokens, and their lower triangle
+    // Right sides, two tiles of 16 columns a wave at a time: K's (filled up to dk16 with zeros), then V's.  The first two are
+    // asked for here, ahead of all else.
+    const size_t ldv = (size_t)a.H * a.dv;
+    const int cts = (p.dk16 + p.dv16) / 16;
+    int ct0 = wave, c[2];
+    bool is_k[2], in[2];
+    f32x4 X[2][4];
+    auto ask = [&]() {
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            const int ct = min(ct0 + u * 4, cts - 1);
+            is_k[u] = ct * 16 < p.dk16;
+            c[u] = ct * 16 - (is_k[u] ? 0 : p.dk16) + r16;
+            in[u] = c[u] < (is_k[u] ? a.d : a.dv);
+            const float* src = is_k[u] ? kp + (in[u] ? c[u] : 0) : a.v.p + (size_t)t0 * ldv + (size_t)h * a.dv + (in[u] ? c[u] : 0);
+            const size_t ld = is_k[u] ? ldk : ldv;
+#pragma unroll
+            for (int b = 0; b < 4; ++b)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) X[u][b][i] = src[(size_t)min(b * 16 + grp * 4 + i, n - 1) * ld];
+        }
+    };
+    ask();
     f32x4 acc[3];
 #pragma unroll
     for (int u = 0; u < 3; ++u) acc[u] = (f32x4){0.f, 0.f, 0.f, 0.f};
     for (int c0 = 0; c0 < a.d; c0 += SL) {
+        Slice ks;
+        ask_slice(ks, kp, ldk, c0, n, a.d);
         if (c0) __syncthreads();
-        load_slice(Ks, kp, ldk, c0, n, a.d);
+        put_slice(Ks, ks, c0, n, a.d);
         __syncthreads();
+        const float e = expf(Ls[CH - 1] - Ls[lane]);  // (the sums stay as they are beyond the chunk's end)
+        for (int c = wave; c < min(SL, p.dk16 - c0); c += 4) p.Kt[(at * p.dk16 + c0 + c) * CH + lane] = e * Ks[lane * LDP + c];
 #pragma unroll
         for (int u = 0; u < 3; ++u) {
             const int tile = wave + u * 4;
@@ -577,6 +659,7 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaChunkArgs p) {
             }
         }
     }
+    if (tid == 0) p.total[at] = expf(Ls[CH - 1]);
 #pragma unroll
     for (int u = 0; u < 3; ++u) {
         const int tile = wave + u * 4;
@@ -606,161 +689,159 @@ __global__ __launch_bounds__(256) void delta_solve_kernel(DeltaChunkArgs p) {
         for (int i = 0; i < 16; ++i) D[i * LDP + lane] = x[i];
     }
     __syncthreads();
-    // Right sides, 16 columns a wave at a time: K's (filled up to dk16 with zeros), then V's.  A block of 16 solved rows is an
-    // accumulator, which serves the blocks below as an operand as it is (see delta_pass_kernel).
-    const size_t ldv = (size_t)a.H * a.dv;
-    for (int ct = wave; ct < (p.dk16 + p.dv16) / 16; ct += 4) {
-        const bool is_k = ct * 16 < p.dk16;
-        const int c = is_k ? ct * 16 + r16 : ct * 16 - p.dk16 + r16;
-        const bool in = c < (is_k ? a.d : a.dv);
-        const float* src = is_k ? kp + (in ? c : 0) : a.v.p + (size_t)t0 * ldv + (size_t)h * a.dv + (in ? c : 0);
-        const size_t ld = is_k ? ldk : ldv;
-        f32x4 X[4];
+    // A block of 16 solved rows is an accumulator, which serves the blocks below as an operand as it is (see delta_pass_kernel).
+    for (; ct0 < cts; ct0 += 8) {
+        if (ct0 != wave) ask();
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
+        for (int u = 0; u < 2; ++u)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int r = b * 16 + grp * 4 + i;
-                const float v = src[(size_t)min(r, n - 1) * ld];
-                X[b][i] = in ? v * (bs[r] * (is_k ? expf(Ls[r]) : 1.f)) : 0.f;  // (beta is zero beyond the chunk's end)
-            }
+            for (int b = 0; b < 4; ++b)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int r = b * 16 + grp * 4 + i;
+                    X[u][b][i] = in[u] ? X[u][b][i] * (bs[r] * (is_k[u] ? expf(Ls[r]) : 1.f)) : 0.f;  // (beta is zero beyond the chunk's end)
+                }
 #pragma unroll
         for (int b = 0; b < 4; ++b) {
             if (b >= used) continue;
-            f32x4 R = X[b];
 #pragma unroll
             for (int e = 0; e < b; ++e) {
                 const f32x4 m = *reinterpret_cast<const f32x4*>(&As[(b * 16 + r16) * LDP + e * 16 + grp * 4]);
 #pragma unroll
-                for (int i = 0; i < 4; ++i) R = mfma_f32(-m[i], X[e][i], R);
+                for (int i = 0; i < 4; ++i)
+#pragma unroll
+                    for (int u = 0; u < 2; ++u) X[u][b] = mfma_f32(-m[i], X[u][e][i], X[u][b]);
             }
             const f32x4 m = *reinterpret_cast<const f32x4*>(&As[(b * 16 + r16) * LDP + b * 16 + grp * 4]);
-            f32x4 Y = (f32x4){0.f, 0.f, 0.f, 0.f};
+            f32x4 Y[2] = {(f32x4){0.f, 0.f, 0.f, 0.f}, (f32x4){0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-            for (int i = 0; i < 4; ++i) Y = mfma_f32(m[i], R[i], Y);
-            X[b] = Y;
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int u = 0; u < 2; ++u) Y[u] = mfma_f32(m[i], X[u][b][i], Y[u]);
+#pragma unroll
+            for (int u = 0; u < 2; ++u) X[u][b] = Y[u];
         }
-        float* dst = is_k ? p.W + ((size_t)t0 * a.H + h) * p.dk16 + c : p.U0 + (size_t)t0 * ldv + (size_t)h * a.dv + c;
-        const size_t ldw = is_k ? (size_t)a.H * p.dk16 : ldv;
+        // tokens beyond the chunk's end and columns beyond the head came out as zeros
 #pragma unroll
-        for (int b = 0; b < 4; ++b)
+        for (int u = 0; u < 2; ++u) {
+            if (ct0 + u * 4 >= cts) continue;
+            if (is_k[u]) {
+                float* dst = p.W + at * CH * p.dk16 + c[u];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int r = b * 16 + grp * 4 + i;
-                if (r < n && (is_k || in)) dst[(size_t)r * ldw] = X[b][i];
+                for (int b = 0; b < 4; ++b)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) dst[(size_t)(b * 16 + grp * 4 + i) * p.dk16] = X[u][b][i];
+            } else {
+                float* dst = p.U0 + (at * p.dv16 + c[u]) * CH + grp * 4;
+#pragma unroll
+                for (int b = 0; b < 4; ++b) *reinterpret_cast<f32x4*>(dst + b * 16) = X[u][b];
             }
+        }
     }
 }
 
 // A block walks a request's chunks for one head and 16 value channels.  Wave w holds the state's rows of the 16-wide tiles
 // w * KT .. w * KT + KT - 1 as accumulators, which serve as operands as they are: lane (grp, r16) holds rows grp * 4 + i of
 // column r16, and supplies them as the four steps i of a product over those rows.
+// FULL: every wave's tiles lie within the head.  Operands are asked for a chunk ahead, into one of two sets of registers in
+// turn, and no load or store of the loop stands behind a condition.
 template <int KT>
+struct PassOperands {
+    f32x4 W[4][KT], K[KT][4], U[4];
+    float g;
+};
+
+template <int KT, bool FULL>
 __global__ __launch_bounds__(256) void delta_pass_kernel(DeltaChunkArgs p) {
     const StateArgs& a = p.a;
     __shared__ f32x4 part[2][4][4][64];
-    const int s = blockIdx.z, h = blockIdx.y, n0 = blockIdx.x * 16, kh = h / (a.H / a.G);
+    // heads first: the blocks of one head, which read the same W and k, lie on one XCD where the heads are a multiple of 8
+    const int s = blockIdx.z, h = blockIdx.x, n0 = blockIdx.y * 16;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
-    const int q0 = a.seq_q_start[s], len = a.seq_q_len[s];
+    const int len = a.seq_q_len[s];
     if (len <= 0) return;
     const int col = n0 + r16;
     const bool col_in = col < a.dv;
     float* st = a.state + ((size_t)a.seq_slot[s] * a.H + h) * a.d * a.dvp;
-    const int base = piece_base(s, CH, a.seq_q_start);
     f32x4 S[KT];
-    int k0[KT];
+    int k0[KT], kk[KT];
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt) {
         k0[kt] = (wave * KT + kt) * 16;
+        kk[kt] = FULL ? k0[kt] : min(k0[kt], p.dk16 - 16);  // a tile beyond the head reads its last one; its state stays zero
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int k = k0[kt] + grp * 4 + i;
             S[kt][i] = (k < a.d && col_in) ? st[(size_t)k * a.dvp + col] : 0.f;
         }
     }
-    f32x4 Wf[4][KT], Kf[KT][4], Uf[4];
-    float lsum = 0.f;
-    const size_t ldk = (size_t)a.G * a.d, ldu = (size_t)a.H * a.dv;
-    auto fetch = [&](int ch) {  // a chunk's operands; rows beyond its end and channels beyond the head are zeros
-        const int t0 = q0 + ch * CH, n = min(CH, len - ch * CH);
-        lsum = decay_sums(a.decay, t0, n, a.H, h, lane);
+    const int nch = (len + CH - 1) / CH;
+    const size_t at0 = (size_t)piece_base(s, CH, a.seq_q_start) * a.H + h, step = a.H;
+    PassOperands<KT> A, B;
+    auto fetch = [&](PassOperands<KT>& o, int ch) {
+        const size_t at = at0 + ch * step;
+        o.g = p.total[at];
+        const float* wp = p.W + (at * CH + r16) * p.dk16 + grp * 4;
+        const float* kp = p.Kt + (at * p.dk16 + r16) * CH + grp * 4;
+        const float* up = p.U0 + (at * p.dv16 + col) * CH + grp * 4;
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt) o.W[rt][kt] = *reinterpret_cast<const f32x4*>(wp + (size_t)rt * 16 * p.dk16 + kk[kt]);
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) {
-            const int r = rt * 16 + r16;
+            o.U[rt] = *reinterpret_cast<const f32x4*>(up + rt * 16);
 #pragma unroll
-            for (int kt = 0; kt < KT; ++kt) {
-                Wf[rt][kt] = (f32x4){0.f, 0.f, 0.f, 0.f};
-                if (r < n && k0[kt] < p.dk16)
-                    Wf[rt][kt] = *reinterpret_cast<const f32x4*>(p.W + ((size_t)(t0 + r) * a.H + h) * p.dk16 + k0[kt] + grp * 4);
-            }
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int j = rt * 16 + grp * 4 + i;
-                const bool row = j < n;
-                Uf[rt][i] = (row && col_in) ? p.U0[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] : 0.f;
-#pragma unroll
-                for (int kt = 0; kt < KT; ++kt) {
-                    const int k = k0[kt] + r16;
-                    Kf[kt][rt][i] = (row && k < a.d) ? a.k.p[(size_t)(t0 + j) * ldk + (size_t)kh * a.d + k] : 0.f;
-                }
-            }
+            for (int kt = 0; kt < KT; ++kt) o.K[kt][rt] = *reinterpret_cast<const f32x4*>(kp + (size_t)kk[kt] * CH + rt * 16);
         }
     };
-    const int nch = (len + CH - 1) / CH;
-    fetch(0);
-    for (int ch = 0; ch < nch; ++ch) {
-        const int t0 = q0 + ch * CH, n = min(CH, len - ch * CH), buf = ch & 1;
-        // the state before the chunk, for the kernel that makes the outputs
-        float* sb = p.Sb + ((size_t)(base + ch) * a.H + h) * p.dk16 * p.dv16 + col;
-#pragma unroll
-        for (int kt = 0; kt < KT; ++kt)
-            if (k0[kt] < p.dk16) {
-#pragma unroll
-                for (int i = 0; i < 4; ++i) sb[(size_t)(k0[kt] + grp * 4 + i) * p.dv16] = S[kt][i];
-            }
+    auto chunk = [&](PassOperands<KT>& cur, PassOperands<KT>& next, int ch, int buf) {
+        const size_t at = at0 + ch * step;
+        fetch(next, min(ch + 1, nch - 1));
+        __builtin_amdgcn_sched_barrier(0);  // the loads go out ahead of the products, not among them
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) {
             f32x4 ws = (f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) ws = mfma_f32(Wf[rt][kt][i], S[kt][i], ws);
+                for (int i = 0; i < 4; ++i) ws = mfma_f32(cur.W[rt][kt][i], S[kt][i], ws);
             part[buf][wave][rt][lane] = ws;
         }
-        const float l = lsum, total = __shfl(l, 63, WAVE), gall = expf(total), e = expf(total - l);
-        f32x4 Us[4], Kc[KT][4];
+        // the state before the chunk, for the kernel that makes the outputs
 #pragma unroll
-        for (int rt = 0; rt < 4; ++rt) {
-            Us[rt] = Uf[rt];
-#pragma unroll
-            for (int kt = 0; kt < KT; ++kt) Kc[kt][rt] = Kf[kt][rt];
-        }
+        for (int kt = 0; kt < KT; ++kt)
+            if (FULL || k0[kt] < p.dk16) *reinterpret_cast<f32x4*>(p.Sb + (at * p.dv16 + col) * p.dk16 + k0[kt] + grp * 4) = S[kt];
         __syncthreads();  // the waves' shares of W S are in LDS (the other half was read before they were written)
-        if (ch + 1 < nch) fetch(ch + 1);
+        f32x4 own = cur.U[0];
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) {
             f32x4 ws = part[buf][0][rt][lane];
 #pragma unroll
             for (int w = 1; w < 4; ++w) ws += part[buf][w][rt][lane];
-            Us[rt] -= ws;
-            if (rt == wave && col_in) {
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const int j = rt * 16 + grp * 4 + i;
-                    if (j < n) p.U[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] = Us[rt][i];
-                }
-            }
-#pragma unroll
-            for (int i = 0; i < 4; ++i) Us[rt][i] *= __shfl(e, rt * 16 + grp * 4 + i, WAVE);
+            cur.U[rt] -= ws;
+            own = rt == wave ? cur.U[rt] : own;
         }
+        *reinterpret_cast<f32x4*>(p.U + (at * p.dv16 + col) * CH + wave * 16 + grp * 4) = own;  // a wave leaves a quarter
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt) {
-            S[kt] *= gall;
+            S[kt] *= cur.g;
+            if (!FULL && k0[kt] >= p.dk16)
 #pragma unroll
-            for (int rt = 0; rt < 4; ++rt)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) S[kt] = mfma_f32(Kc[kt][rt][i], Us[rt][i], S[kt]);
+                for (int rt = 0; rt < 4; ++rt) cur.K[kt][rt] = (f32x4){0.f, 0.f, 0.f, 0.f};
         }
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int kt = 0; kt < KT; ++kt) S[kt] = mfma_f32(cur.K[kt][rt][i], cur.U[rt][i], S[kt]);
+    };
+    fetch(A, 0);
+    for (int ch = 0; ch < nch; ch += 2) {
+        chunk(A, B, ch, 0);
+        if (ch + 1 >= nch) break;
+        chunk(B, A, ch + 1, 1);
     }
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt)
@@ -783,10 +864,10 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
     const int n = min(left, CH), t0 = a.seq_q_start[pc.s] + pc.first, h = blockIdx.y, kh = h / (a.H / a.G);
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, grp = lane >> 4;
     const int used = (n + 15) / 16, tiles = used * (used + 1) / 2;
-    const size_t ldk = (size_t)a.G * a.d, ldu = (size_t)a.H * a.dv;
+    const size_t ldk = (size_t)a.G * a.d;
     const float* qp = a.q.p + (size_t)t0 * ldk + (size_t)kh * a.d;
     const float* kp = a.k.p + (size_t)t0 * ldk + (size_t)kh * a.d;
-    const float* sb = p.Sb + ((size_t)blockIdx.x * a.H + h) * p.dk16 * p.dv16;
+    const size_t at = (size_t)blockIdx.x * a.H + h;
     if (wave == 0) Ls[lane] = decay_sums(a.decay, t0, n, a.H, h, lane);
     f32x4 O[4][CT], P[3];
 #pragma unroll
@@ -796,21 +877,19 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
 #pragma unroll
         for (int c = 0; c < CT; ++c) O[rt][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
     for (int c0 = 0; c0 < a.d; c0 += SL) {
-        f32x4 B[SL / 16][CT];  // the state's rows c0 .. c0 + SL of this wave's columns
+        Slice qs, ks;
+        ask_slice(qs, qp, ldk, c0, n, a.d);
+        ask_slice(ks, kp, ldk, c0, n, a.d);
+        f32x4 B[SL / 16][CT];  // the state's rows c0 .. c0 + SL of this wave's columns (rows beyond it meet zeros of q)
 #pragma unroll
         for (int kk = 0; kk < SL / 16; ++kk)
 #pragma unroll
-            for (int c = 0; c < CT; ++c) {
-                const int col = (wave + 4 * c) * 16 + r16;
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const int k = c0 + kk * 16 + grp * 4 + i;
-                    B[kk][c][i] = (k < p.dk16 && col < p.dv16) ? sb[(size_t)k * p.dv16 + col] : 0.f;
-                }
-            }
+            for (int c = 0; c < CT; ++c)
+                B[kk][c] = *reinterpret_cast<const f32x4*>(p.Sb + (at * p.dv16 + min((wave + 4 * c) * 16, p.dv16 - 16) + r16) * p.dk16 +
+                                                           min(c0 + kk * 16, p.dk16 - 16) + grp * 4);
         if (c0) __syncthreads();
-        load_slice(Qs, qp, ldk, c0, n, a.d);
-        load_slice(Ks, kp, ldk, c0, n, a.d);
+        put_slice(Qs, qs, c0, n, a.d);
+        put_slice(Ks, ks, c0, n, a.d);
         __syncthreads();
 #pragma unroll
         for (int u = 0; u < 3; ++u) {
@@ -866,14 +945,8 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
 #pragma unroll
     for (int jt = 0; jt < 4; ++jt)
 #pragma unroll
-        for (int c = 0; c < CT; ++c) {
-            const int col = (wave + 4 * c) * 16 + r16;
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int j = jt * 16 + grp * 4 + i;
-                Uf[jt][c][i] = (j < n && col < a.dv) ? p.U[(size_t)(t0 + j) * ldu + (size_t)h * a.dv + col] : 0.f;
-            }
-        }
+        for (int c = 0; c < CT; ++c)
+            Uf[jt][c] = *reinterpret_cast<const f32x4*>(p.U + (at * p.dv16 + min((wave + 4 * c) * 16, p.dv16 - 16) + r16) * CH + jt * 16 + grp * 4);
     __syncthreads();
 #pragma unroll
     for (int rt = 0; rt < 4; ++rt) {
@@ -887,6 +960,25 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
                 for (int i = 0; i < 4; ++i) O[rt][c] = mfma_f32(x[i], Uf[jt][c][i], O[rt][c]);
         }
     }
+    float nw[CT];
+#pragma unroll
+    for (int c = 0; c < CT; ++c) nw[c] = a.norm[min((wave + 4 * c) * 16 + r16, a.dv - 1)];
+    // the gates of this lane's places, every load on one straight path
+    f32x4 Z[4][CT];
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int c = 0; c < CT; ++c) Z[rt][c] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int q = 0; q < a.gate.n; ++q) {
+        const float* gp = a.gate.p + q * a.gate.stride + (size_t)t0 * a.gate.ld + a.g_col + h * a.dv;
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+            for (int c = 0; c < CT; ++c)
+#pragma unroll
+                for (int ii = 0; ii < 4; ++ii)
+                    Z[rt][c][ii] += gp[(size_t)min(rt * 16 + grp * 4 + ii, n - 1) * a.gate.ld + min((wave + 4 * c) * 16 + r16, a.dv - 1)];
+    }
     // the heads' norms: a row's squares over this wave's columns, then over the waves
 #pragma unroll
     for (int rt = 0; rt < 4; ++rt)
@@ -894,7 +986,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
         for (int ii = 0; ii < 4; ++ii) {
             float ss = 0.f;
 #pragma unroll
-            for (int c = 0; c < CT; ++c) ss += O[rt][c][ii] * O[rt][c][ii];  // columns beyond dv are zeros
+            for (int c = 0; c < CT; ++c) ss += (wave + 4 * c) * 16 + r16 < a.dv ? O[rt][c][ii] * O[rt][c][ii] : 0.f;
 #pragma unroll
             for (int o = 1; o < 16; o <<= 1) ss += __shfl_xor(ss, o, WAVE);
             if (r16 == 0) rows[wave][rt * 16 + grp * 4 + ii] = ss;
@@ -913,7 +1005,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaChunkArgs p) {
                 const int col = (wave + 4 * c) * 16 + r16;
                 if (col < a.dv)
                     a.out[(size_t)t * a.ld_out + h * a.dv + col] =
-                        from_f32<elem_t>(O[rt][c][ii] * inv * a.norm[col] * silu_f(sum_at(a.gate, t, a.g_col + h * a.dv + col)));
+                        from_f32<elem_t>(O[rt][c][ii] * inv * nw[c] * silu_f(Z[rt][c][ii]));
             }
         }
     if (h == 0)
@@ -927,7 +1019,11 @@ using namespace ms;
 extern "C" int ms_gated_state_max_taps() { return MAX_TAPS; }
 extern "C" int ms_gated_state_max_dim() { return MAX_DIM; }
 extern "C" int ms_gated_state_max_rank() { return 1536; }  // eight rows of it lie in LDS
-extern "C" int ms_delta_chunk() { return CH; }
+// floats of the workspace of the delta rule's chunks
+extern "C" long ms_delta_work(int T, int S, int H, int d, int dv) {
+    const long dk16 = ceil_div(d, 16) * 16, dv16 = ceil_div(dv, 16) * 16;
+    return (long)(T / CH + S) * H * (2 * CH * (dk16 + dv16) + dk16 * dv16 + 1);
+}
 
 // in: float [n_partials, T, ld].  many: requests of several rows may be among the step's (their states are then brought up
 // to date by a second launch).
@@ -1063,27 +1159,35 @@ extern "C" int ms_gated_linear(const float* rows, int n_partials, int ld, int q_
 
 // The gated delta rule.  q, k float [T, G * d] (unit vectors, q scaled), v float [T, H * dv], lg and beta float [T, H] as
 // ms_delta_rows leaves them; gate: columns g_col on of float [n_partials, T, ld].  single: every request has one row; else
-// W float [T, H, dk16], U0 and U float [T, H, dv] and Sb float [T / 64 + S, H, dk16, dv16] are the workspace.
+// work float [(T / 64 + S) H (2 * 64 dk16 + 2 * 64 dv16 + dk16 dv16 + 1)] (ms_delta_work) is the workspace.
 extern "C" int ms_gated_delta(const float* q, const float* k, const float* v, const float* lg, const float* beta, const float* gate,
                               int n_partials, int ld, int g_col, const float* norm, float eps, float* state, const int* seq_q_start,
                               const int* seq_q_len, const int* seq_slot, int S, void* out, int ld_out, int T, int H, int G, int d, int dv,
-                              int dvp, int single, float* W, float* U0, float* U, float* Sb, hipStream_t stream) {
+                              int dvp, int single, float* work, hipStream_t stream) {
     const Sums qs{q, 1, 0, G * d}, ks{k, 1, 0, G * d}, vs{v, 1, 0, H * dv}, gs{gate, n_partials, (size_t)T * ld, ld};
     const StateArgs a{qs, ks, vs, 0, 0, 0, 1.0f, lg, beta, gs, g_col, norm, eps, state, seq_q_start, seq_q_len, seq_slot, S,
                       (elem_t*)out, ld_out, T, H, G, d, dv, dvp};
     MS_REQUIRE(n_partials > 0 && beta, "gated delta: no rows");
     if (int rc = check_state(a, "gated delta")) return rc;
     if (single) return launch_step<true>(a, stream);
-    MS_REQUIRE(W && U0 && U && Sb && S <= 65535, "gated delta: chunks of %d need their workspace", CH);
-    MS_REQUIRE((reinterpret_cast<uintptr_t>(W)) % 16 == 0, "gated delta: the workspace must be 16-byte aligned");
-    const DeltaChunkArgs p{a, W, U0, U, Sb, ceil_div(d, 16) * 16, ceil_div(dv, 16) * 16};
-    const int numbers = T / CH + S;
+    MS_REQUIRE(work && S <= 65535, "gated delta: chunks of %d need their workspace", CH);
+    MS_REQUIRE((reinterpret_cast<uintptr_t>(work)) % 16 == 0, "gated delta: the workspace must be 16-byte aligned");
+    const int numbers = T / CH + S, dk16 = ceil_div(d, 16) * 16, dv16 = ceil_div(dv, 16) * 16;
+    const size_t nh = (size_t)numbers * H, kf = nh * CH * dk16, vf = nh * CH * dv16;
+    const DeltaChunkArgs p{a, work, work + kf, work + 2 * kf, work + 2 * kf + vf, work + 2 * kf + 2 * vf, work + 2 * kf + 2 * vf + nh * dk16 * dv16,
+                           dk16, dv16};
     hipLaunchKernelGGL(delta_solve_kernel, dim3(numbers, H), dim3(256), 0, stream, p);
     if (int rc = check_launch("gated delta, chunks solved")) return rc;
-    const dim3 grid(ceil_div(dv, 16), H, S);
-    if (d <= 64) hipLaunchKernelGGL(delta_pass_kernel<1>, grid, dim3(256), 0, stream, p);
-    else if (d <= 128) hipLaunchKernelGGL(delta_pass_kernel<2>, grid, dim3(256), 0, stream, p);
-    else hipLaunchKernelGGL(delta_pass_kernel<4>, grid, dim3(256), 0, stream, p);
+    const dim3 grid(H, ceil_div(dv, 16), S);
+#define MS_PASS(KT)                                                                                                         \
+    do {                                                                                                                    \
+        if (dk16 == 64 * KT) hipLaunchKernelGGL((delta_pass_kernel<KT, true>), grid, dim3(256), 0, stream, p);              \
+        else hipLaunchKernelGGL((delta_pass_kernel<KT, false>), grid, dim3(256), 0, stream, p);                             \
+    } while (0)
+    if (d <= 64) MS_PASS(1);
+    else if (d <= 128) MS_PASS(2);
+    else MS_PASS(4);
+#undef MS_PASS
     if (int rc = check_launch("gated delta, states between chunks")) return rc;
     if (dv <= 64) hipLaunchKernelGGL(delta_out_kernel<1>, dim3(numbers, H), dim3(256), 0, stream, p);
     else if (dv <= 128) hipLaunchKernelGGL(delta_out_kernel<2>, dim3(numbers, H), dim3(256), 0, stream, p);

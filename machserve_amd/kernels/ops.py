@@ -1599,16 +1599,14 @@ class HipOps:
         if single and S != T:
             raise KernelError(f"gated delta: {T} rows of {S} requests are not single rows")
         out = torch.empty((T, out_cols), dtype=self.dtype, device=q.device)
-        W = U0 = U = Sb = None
+        work = None
         if not single:
-            dk16, dv16 = -(-d // 16) * 16, -(-dv // 16) * 16
-            new = lambda *shape: torch.empty(shape, dtype=torch.float32, device=q.device)
-            W, U0, U = new(T, H, dk16), new(T, H, dv), new(T, H, dv)
-            Sb = new(T // lib.ms_delta_chunk() + S, H, dk16, dv16)
+            lib.ms_delta_work.restype = ctypes.c_long
+            work = torch.empty((lib.ms_delta_work(_c_int(T), _c_int(S), _c_int(H), _c_int(d), _c_int(dv)),), dtype=torch.float32, device=q.device)
         self._check(lib, lib.ms_gated_delta(
             _ptr(q), _ptr(k), _ptr(v), _ptr(lg), _ptr(beta), _ptr(sums), _c_int(P), _c_int(N), _c_int(gate_col), _ptr(norm_w), _c_float(eps), _ptr(state),
             _ptr(seq_q_start), _ptr(seq_q_len), _ptr(seq_slot), _c_int(S), _ptr(out), _c_int(out_cols), _c_int(T), _c_int(H), _c_int(G), _c_int(d),
-            _c_int(dv), _c_int(dvp), _c_int(int(single)), _ptr(W), _ptr(U0), _ptr(U), _ptr(Sb), self._stream()))
+            _c_int(dv), _c_int(dvp), _c_int(int(single)), _ptr(work), self._stream()))
         return out
 
     # ------------------------------------------------------------------ sampling
