@@ -248,6 +248,74 @@ __global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ x, co
     for (int c = threadIdx.x; c < d; c += 256) dst[c] += vals[c] * inv * w[c];
 }
 
+// A branch's norm behind it and the next branch's norm ahead of it, in one pass over the row:
+// x[t, :] += y / rms(y) * w  with y as norm_add_kernel has it,  then  out[t, :] = x / rms(x) * w2 in the element type.
+// For widths that are a multiple of four and at most 1024 * G, and up to NP sums a branch: a thread owns G groups of four
+// columns and asks for everything the row needs before it uses the first value (sums beyond the last one read the last one
+// again and count for nothing).
+template <int G, int NP, bool PAIR>
+__global__ __launch_bounds__(256) void norm_add_norm_kernel(float* __restrict__ x, const float* __restrict__ pa, int na, float fa,
+                                                            const float* __restrict__ pb, int nb, float fb, size_t partial_stride,
+                                                            const float* __restrict__ w, float eps, const float* __restrict__ w2, float eps2,
+                                                            elem_t* __restrict__ out, int d) {
+    arguments_now(x, pa, na, fa, pb, nb, fb, partial_stride, w, eps, w2, eps2, out, d);
+    __shared__ float scratch[4];
+    const size_t r = blockIdx.x;
+    const int ng = d / 4;
+    f32x4* row = reinterpret_cast<f32x4*>(x + r * d);
+    const f32x4* sa = reinterpret_cast<const f32x4*>(pa + r * d);
+    const f32x4* sb = PAIR ? reinterpret_cast<const f32x4*>(pb + r * d) : nullptr;
+    const size_t stride4 = partial_stride / 4;
+    f32x4 v[G], wv[G], w2v[G], qa[NP][G], qb[PAIR ? NP : 1][G];
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        const int c4 = threadIdx.x + g * 256, at = c4 < ng ? c4 : 0;  // a group beyond the row reads group 0 and is dropped
+        v[g] = row[at];
+        wv[g] = reinterpret_cast<const f32x4*>(w)[at];
+        w2v[g] = reinterpret_cast<const f32x4*>(w2)[at];
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+            qa[p][g] = sa[(size_t)min(p, na - 1) * stride4 + at];
+            if constexpr (PAIR) qb[p][g] = sb[(size_t)min(p, nb - 1) * stride4 + at];
+        }
+    }
+    float ss = 0.f;
+    f32x4 y[G];
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        f32x4 a = qa[0][g];
+#pragma unroll
+        for (int p = 1; p < NP; ++p) a += qa[p][g] * (p < na ? 1.f : 0.f);
+        y[g] = a * fa;
+        if constexpr (PAIR) {
+            f32x4 b = qb[0][g];
+#pragma unroll
+            for (int p = 1; p < NP; ++p) b += qb[p][g] * (p < nb ? 1.f : 0.f);
+            y[g] += b * fb;
+        }
+        if (threadIdx.x + g * 256 < ng) ss += y[g].x * y[g].x + y[g].y * y[g].y + y[g].z * y[g].z + y[g].w * y[g].w;
+    }
+    ss = block_sum<256>(ss, scratch);
+    const float inv = 1.0f / sqrtf(ss / (float)d + eps);
+    float s2 = 0.f;
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        v[g] += y[g] * inv * wv[g];
+        if (threadIdx.x + g * 256 < ng) s2 += v[g].x * v[g].x + v[g].y * v[g].y + v[g].z * v[g].z + v[g].w * v[g].w;
+    }
+    s2 = block_sum<256>(s2, scratch);
+    const float inv2 = 1.0f / sqrtf(s2 / (float)d + eps2);
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+        const int c4 = threadIdx.x + g * 256;
+        if (c4 >= ng) continue;
+        row[c4] = v[g];
+        const f32x4 o = v[g] * w2v[g] * inv2;
+        typedef elem_t out4_t __attribute__((ext_vector_type(4)));
+        *reinterpret_cast<out4_t*>(out + r * d + (size_t)c4 * 4) = (out4_t){from_f32<elem_t>(o.x), from_f32<elem_t>(o.y), from_f32<elem_t>(o.z), from_f32<elem_t>(o.w)};
+    }
+}
+
 // x[t, :] += first[t, :] (null: nothing) + row: what comes ahead of a pass over looped layers
 __global__ __launch_bounds__(256) void open_pass_kernel(float* __restrict__ x, const float* __restrict__ first, const float* __restrict__ row,
                                                         int d, size_t n) {
@@ -714,6 +782,37 @@ extern "C" int ms_norm_add_weighted(float* x, const float* pa, int na, float fa,
     hipLaunchKernelGGL(norm_add_kernel<true>, dim3(T), dim3(256), (size_t)d * sizeof(float), stream, x, pa, na, (size_t)T * d, w, d, eps,
                        (const float*)nullptr, fa, pb, nb, fb);
     return check_launch("norm_add_weighted");
+}
+
+// Whether ms_norm_add_norm takes rows of d numbers with na and nb sums (nb 0: one branch).
+extern "C" int ms_norm_add_norm_takes(int d, int na, int nb) {
+    const int g = d % 4 == 0 ? (d <= 1024 ? 1 : (d <= 2048 ? 2 : (d <= 4096 ? 4 : 0))) : 0, most = na > nb ? na : nb;
+    return g > 0 && na >= 1 && most * g * (nb ? 2 : 1) <= 16 && most <= 8;
+}
+
+// x += rmsnorm(fa sum(pa) + fb sum(pb)) * w (pb null: the first branch alone), out = rmsnorm(x) * w2 in the element type
+extern "C" int ms_norm_add_norm(float* x, const float* pa, int na, float fa, const float* pb, int nb, float fb, const float* w, float eps,
+                                const float* w2, float eps2, void* out, int T, int d, hipStream_t stream) {
+    MS_REQUIRE(T > 0 && d > 0 && ms_norm_add_norm_takes(d, na, pb ? nb : 0), "norm_add_norm: T=%d d=%d with %d and %d sums", T, d, na, nb);
+    MS_REQUIRE(x && pa && w && w2 && out && (pb == nullptr) == (nb == 0), "norm_add_norm: a buffer is missing");
+    MS_REQUIRE((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(pa) | reinterpret_cast<uintptr_t>(pb) | reinterpret_cast<uintptr_t>(w) |
+                reinterpret_cast<uintptr_t>(w2) | reinterpret_cast<uintptr_t>(out)) % 16 == 0, "norm_add_norm: buffers must be 16-byte aligned");
+    const size_t ps = (size_t)T * d;
+    const int groups = d <= 1024 ? 1 : (d <= 2048 ? 2 : 4), most = na > nb ? na : nb;
+#define MS_NAN(G_, NP_, PAIR_)                                                                                                            \
+    hipLaunchKernelGGL((norm_add_norm_kernel<G_, NP_, PAIR_>), dim3(T), dim3(256), 0, stream, x, pa, na, fa, pb, nb, fb, ps, w, eps, w2, eps2, \
+                       (elem_t*)out, d)
+    if (pb == nullptr) {
+        if (groups == 1) { if (most == 1) MS_NAN(1, 1, false); else if (most == 2) MS_NAN(1, 2, false); else if (most <= 4) MS_NAN(1, 4, false); else MS_NAN(1, 8, false); }
+        else if (groups == 2) { if (most == 1) MS_NAN(2, 1, false); else if (most == 2) MS_NAN(2, 2, false); else if (most <= 4) MS_NAN(2, 4, false); else MS_NAN(2, 8, false); }
+        else { if (most == 1) MS_NAN(4, 1, false); else if (most == 2) MS_NAN(4, 2, false); else MS_NAN(4, 4, false); }
+    } else {
+        if (groups == 1) { if (most == 1) MS_NAN(1, 1, true); else if (most == 2) MS_NAN(1, 2, true); else if (most <= 4) MS_NAN(1, 4, true); else MS_NAN(1, 8, true); }
+        else if (groups == 2) { if (most == 1) MS_NAN(2, 1, true); else if (most == 2) MS_NAN(2, 2, true); else MS_NAN(2, 4, true); }
+        else { if (most == 1) MS_NAN(4, 1, true); else MS_NAN(4, 2, true); }
+    }
+#undef MS_NAN
+    return check_launch("norm_add_norm");
 }
 
 extern "C" int ms_open_pass(float* x, const float* first, const float* row, int T, int d, hipStream_t stream) {

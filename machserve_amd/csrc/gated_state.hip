@@ -269,18 +269,38 @@ __global__ __launch_bounds__(256) void state_step_kernel(StateArgs a) {
         S[j] = (f32x4){0.f, 0.f, 0.f, 0.f};
         if (col_in && i < a.d) S[j] = *reinterpret_cast<const f32x4*>(st + (size_t)i * a.dvp);
     }
-    const bool live = tid < a.dv;
-    const float vc = live ? sum_at(a.v, t, a.v_col + h * a.dv + tid) : 0.f;
-    const float zc = live ? sum_at(a.gate, t, a.g_col + h * a.dv + tid) : 0.f;
-    float qk = 0.f;
-    for (int i = tid; i < DP; i += 256) {
-        const bool in = i < a.d;
-        const float qv = in ? sum_at(a.q, t, a.q_col + kh * a.d + i) * a.q_scale : 0.f, kv = in ? sum_at(a.k, t, a.k_col + kh * a.d + i) : 0.f;
-        qs[i] = qv;
-        ks[i] = kv;
-        if (!DELTA) ws[i] = in ? a.decay[((size_t)t * a.H + h) * a.d + i] : 0.f;
-        qk += qv * kv;
+    // this thread's numbers of q, k, v and the gate (it drops what lies beyond a head): every load on one straight path
+    const bool live = tid < a.dv, in = tid < a.d;
+    const int ci = min(tid, a.d - 1), cv = min(tid, a.dv - 1);
+    const float alpha = DELTA ? 0.f : a.decay[((size_t)t * a.H + h) * a.d + ci];
+    float vc = 0.f, zc = 0.f, qv = 0.f, kv = 0.f;
+    const float* gp = a.gate.p + (size_t)t * a.gate.ld + a.g_col + h * a.dv + cv;
+    if constexpr (DELTA) {
+        qv = a.q.p[(size_t)t * a.q.ld + a.q_col + kh * a.d + ci];
+        kv = a.k.p[(size_t)t * a.k.ld + a.k_col + kh * a.d + ci];
+        vc = a.v.p[(size_t)t * a.v.ld + a.v_col + h * a.dv + cv];
+#pragma unroll 4
+        for (int p = 0; p < a.gate.n; ++p) zc += gp[p * a.gate.stride];
+    } else {  // columns of the same rows
+        const float* rp = a.q.p + (size_t)t * a.q.ld;
+#pragma unroll 4
+        for (int p = 0; p < a.q.n; ++p) {
+            const float* r = rp + p * a.q.stride;
+            qv += r[a.q_col + kh * a.d + ci];
+            kv += r[a.k_col + kh * a.d + ci];
+            vc += r[a.v_col + h * a.dv + cv];
+            zc += gp[p * a.gate.stride];
+        }
     }
+    qv = in ? qv * a.q_scale : 0.f;
+    kv = in ? kv : 0.f;
+    if (!live) vc = 0.f;
+    if (tid < DP) {
+        qs[tid] = qv;
+        ks[tid] = kv;
+        if (!DELTA) ws[tid] = in ? alpha : 0.f;
+    }
+    float qk = qv * kv;
     const float g = DELTA ? expf(a.decay[(size_t)t * a.H + h]) : 1.f, beta = DELTA ? a.beta[(size_t)t * a.H + h] : 1.f;
     if (!DELTA && tid < W) us[tid] = vc;
     if (DELTA) qk = block_sum<256>(qk, scratch);  // (a barrier: the rows are in LDS)

@@ -1038,6 +1038,27 @@ class HipOps:
         self._check(self._core, self._core.ms_norm_add_weighted(_ptr(x), _ptr(pa), _c_int(pa.shape[0]), _c_float(fa), _ptr(pb), _c_int(pb.shape[0]),
                                                                 _c_float(fb), _ptr(weight), _c_int(T), _c_int(d), _c_float(eps), self._stream()))
 
+    def norm_add_norm_takes(self, d: int, branches) -> bool:
+        """Whether :meth:`norm_add_norm` takes rows of ``d`` numbers with these branches' sums."""
+        counts = [p.shape[0] for p, _ in branches]
+        return len(counts) <= 2 and bool(self._plan("ms_norm_add_norm_takes", d, counts[0], counts[1] if len(counts) > 1 else 0))
+
+    def norm_add_norm(self, x: torch.Tensor, branches, weight: torch.Tensor, eps: float, weight2: torch.Tensor, eps2: float) -> torch.Tensor:
+        """In place ``x += rmsnorm(sum_i f_i sum(p_i)) * weight`` for one or two ``branches`` ``(p_i, f_i)`` with ``p_i`` float32 ``[P, T, d]``;
+        returns ``rmsnorm(x) * weight2`` in the element type: a branch's norm behind it and the next one's ahead of it."""
+        T, d = x.shape
+        self._want(x, torch.float32, "norm_add_norm stream")
+        for p, _ in branches:
+            self._want(p, torch.float32, "norm_add_norm sums", p.shape[0], T, d)
+        self._want(weight, torch.float32, "norm_add_norm weight", d)
+        self._want(weight2, torch.float32, "norm_add_norm weight", d)
+        (pa, fa), (pb, fb) = branches[0], (branches[1] if len(branches) > 1 else (None, 0.0))
+        out = torch.empty((T, d), dtype=self.dtype, device=x.device)
+        self._check(self._core, self._core.ms_norm_add_norm(
+            _ptr(x), _ptr(pa), _c_int(pa.shape[0]), _c_float(fa), _ptr(pb), _c_int(0 if pb is None else pb.shape[0]), _c_float(fb), _ptr(weight),
+            _c_float(eps), _ptr(weight2), _c_float(eps2), _ptr(out), _c_int(T), _c_int(d), self._stream()))
+        return out
+
     def open_pass(self, x: torch.Tensor, first: Optional[torch.Tensor], row: torch.Tensor) -> None:
         """``x += first + row`` in place: the rows of ``first`` (None: nothing) and one row for all, in 32-bit."""
         T, d = x.shape

@@ -110,7 +110,8 @@ class ResidualStream:
     ``add_linear`` does not launch its product at once but when the stream is next read.  With
     few rows the product leaves partial sums (``pending``) that a reading norm may add in its
     own kernel, which saves a pass over the stream; with many rows the product adds to the
-    stream in its epilogue.  A reader that knows nothing of this calls ``value()``.
+    stream in its epilogue.  A branch that is normed on its way out (``add_normed_sums``) is not added at once either: where
+    the next reader is a norm, one kernel adds it and norms the stream.  A reader that knows nothing of this calls ``value()``.
     """
 
     def __init__(self, x: torch.Tensor, ops):
@@ -118,6 +119,7 @@ class ResidualStream:
         self.ops = ops
         self.deferred = None                         # (a, w): x += a @ w.T, not yet launched
         self.pending: Optional[torch.Tensor] = None  # float32 [P, T, width], not yet added
+        self.post = None  # (branches, weight, eps): x += rmsnorm(sum_i f_i sum(p_i)) * weight, not yet added
         self.rounded: Optional[torch.Tensor] = None  # x in the element type, if whoever wrote x left it as well
 
     def add_linear(self, a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> None:
@@ -151,8 +153,29 @@ class ResidualStream:
         self.open()
         self.ops.add_scaled_rows(self.x, h, weights, first, count)
 
+    def add_normed_sums(self, branches, weight: torch.Tensor, eps: float) -> None:
+        """``x += rmsnorm(sum_i f_i sum(p_i)) * weight`` for one or two ``branches`` ``(p_i, f_i)``, ``p_i`` the partial sums of a last
+        product; left to the next reader where the kernels can add it together with that reader's norm."""
+        self.open()
+        self.post = (branches, weight, eps)
+        takes = getattr(self.ops, "norm_add_norm_takes", None)
+        if takes is None or not takes(self.x.shape[1], branches):
+            self._add_post()
+
+    def _add_post(self) -> None:
+        branches, weight, eps = self.post
+        self.post = None
+        if len(branches) == 1 and branches[0][1] == 1.0:
+            self.ops.norm_add(self.x, branches[0][0], weight, eps)
+        else:
+            (pa, fa), (pb, fb) = branches
+            self.ops.norm_add_weighted(self.x, pa, fa, pb, fb, weight, eps)
+
     def launch_deferred(self) -> None:
-        """Launch the product that ``add_linear`` left, if any; its sum may stay pending as partial sums."""
+        """Launch the product that ``add_linear`` left, if any; its sum may stay pending as partial sums.  A normed branch that
+        is still to be added is added."""
+        if self.post is not None:
+            self._add_post()
         if self.deferred is not None:
             a, w = self.deferred
             self.deferred = None

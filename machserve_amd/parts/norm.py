@@ -31,7 +31,10 @@ class RMSNorm(Norm):
 
     def forward(self, stream, rows=None):
         """``rmsnorm(x) * weight`` of the stream with everything added (of its ``rows`` if given), in the
-        element type; partial sums that are pending are added by the norm's own kernel."""
+        element type; what is pending (partial sums, a normed branch) is added by the norm's own kernel."""
+        if stream.post is not None and rows is None:
+            post, stream.post = stream.post, None
+            return stream.ops.norm_add_norm(stream.x, *post, self.weight, self.spec.eps)
         stream.launch_deferred()
         h = stream.ops.rmsnorm(stream.x, self.weight, self.spec.eps, rows, False, stream.pending)
         if rows is None:
@@ -44,10 +47,10 @@ class RMSNorm(Norm):
     def add_normed(self, stream, a, w, bias=None) -> None:
         """``x += rmsnorm(a @ w.T (+ bias)) * weight``: the norm after a branch whose last step is a product.  The product
         leaves its sums in 32-bit, and one kernel adds them up, normalises the row and adds it to the stream."""
-        stream.open()
         if bias is None:
-            stream.ops.norm_add(stream.x, stream.ops.linear_split(a, w), self.weight, self.spec.eps)
+            stream.add_normed_sums([(stream.ops.linear_split(a, w), 1.0)], self.weight, self.spec.eps)
         else:
+            stream.open()
             stream.ops.norm_add_bias(stream.x, stream.ops.linear_split(a, w), bias, self.weight, self.spec.eps)
 
     def add_normed_mean(self, stream, branches, eps) -> None:
@@ -67,10 +70,7 @@ class RMSNorm(Norm):
         fa), ((b, w_b), fb)]`` with each branch the operands of its last product."""
         if len(branches) != 2:
             raise ValueError(f"{len(branches)} branches side by side under a norm: the kernel takes two")
-        ((a, w_a), fa), ((b, w_b), fb) = branches
-        stream.open()
-        ops = stream.ops
-        ops.norm_add_weighted(stream.x, ops.linear_split(a, w_a), float(fa), ops.linear_split(b, w_b), float(fb), self.weight, self.spec.eps)
+        stream.add_normed_sums([(stream.ops.linear_split(*product), float(f)) for product, f in branches], self.weight, self.spec.eps)
 
     def normalise_sum(self, stream, alpha: float, sums, bias=None) -> None:
         """``x <- rmsnorm(alpha x + sum(sums) (+ bias)) * weight``: the norm behind a residual sum.  ``sums`` float32 ``[P, T,
@@ -122,10 +122,17 @@ class LayerNorm(Norm):
 
 
 class PendingRMSNorm(PendingNorm):
-    """The RMS norm left to its reader's first product, folded into it where the kernels take the shape."""
+    """The RMS norm left to its reader's first product, folded into it where the kernels take the shape.  Where a normed branch
+    is still to be added to the stream and the product does not take the norm, the two norms are one kernel."""
+
+    def _post_goes_first(self, n: int) -> bool:
+        stream = self.stream
+        return stream.post is not None and not stream.ops.norm_folds_into(stream.x.shape[0], n, stream.x.shape[1], 0)
 
     def linear_split(self, w):
         stream, ops, weight, eps = self.stream, self.stream.ops, self.norm.weight, self.norm.spec.eps
+        if self._post_goes_first(w.shape[0]):
+            return ops.linear_split(self.tensor(), w)
         stream.launch_deferred()
         T, K = stream.x.shape
         P = 0 if stream.pending is None else stream.pending.shape[0]
@@ -138,6 +145,8 @@ class PendingRMSNorm(PendingNorm):
 
     def linear_swiglu(self, w_gate_up, intermediate, activation="silu"):
         stream, ops, weight, eps = self.stream, self.stream.ops, self.norm.weight, self.norm.spec.eps
+        if self._post_goes_first(w_gate_up.shape[0]):
+            return ops.linear_swiglu(self.tensor(), w_gate_up, intermediate, activation)
         if stream.deferred is not None and stream.pending is None:
             # a product that is still to be added: where the kernels can, it leaves what the norm needs beside its
             # sum, and the gated product applies the norm's factor to its own finished sums

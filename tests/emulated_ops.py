@@ -325,6 +325,14 @@ class EmulatedOps:
         y = fa * pa.sum(0) + fb * pb.sum(0)
         x += y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps)) * weight
 
+    def norm_add_norm_takes(self, d, branches):
+        return d % 4 == 0 and max(p.shape[0] for p, _ in branches) <= 4
+
+    def norm_add_norm(self, x, branches, weight, eps, weight2, eps2):
+        y = sum(f * p.sum(0) for p, f in branches)
+        x += y * (1.0 / torch.sqrt((y * y).sum(-1, keepdim=True) / y.shape[-1] + eps)) * weight
+        return self._r(x * (1.0 / torch.sqrt((x * x).sum(-1, keepdim=True) / x.shape[-1] + eps2)) * weight2)
+
     def open_pass(self, x, first, row):
         if first is not None:
             x += first

@@ -159,6 +159,27 @@ def test_norm_of_two_weighted_branches(d, T):
         close(got, want, torch.float32, f"{na} and {nb} sums", 1e-5)
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d,T", [(48, 5), (256, 70), (1024, 33), (1028, 3), (2048, 9), (4096, 5)])
+def test_norm_behind_a_branch_and_ahead_of_the_next(dtype, d, T):
+    ops, ref = ops_of(dtype), EmulatedOps(dtype)
+    torch.manual_seed(d)
+    w, w2 = torch.randn(d), torch.randn(d)
+    taken = 0
+    for counts, factors in (((1,), (1.0,)), ((2,), (1.0,)), ((3,), (1.0,)), ((8,), (1.0,)), ((9,), (1.0,)), ((1, 1), (1.2, -0.4)), ((2, 1), (0.5, 2.0)), ((3, 4), (1.0, 1.0)), ((1, 7), (2.0, 0.1))):
+        x, branches = torch.randn(T, d) * 2, [(torch.randn(n, T, d), f) for n, f in zip(counts, factors)]
+        if not ops.norm_add_norm_takes(d, branches):
+            continue
+        taken += 1
+        want_x, got_x = x.clone(), dev(x)
+        want = ref.norm_add_norm(want_x, branches, w, 1e-5, w2, 1e-4)
+        got = ops.norm_add_norm(got_x, [(dev(p), f) for p, f in branches], dev(w), 1e-5, dev(w2), 1e-4)
+        close(got_x, want_x, torch.float32, f"stream after {counts}", 1e-5)
+        close(got, want, dtype, f"rows for the next branch after {counts}")
+    assert taken >= 4
+    assert not ops.norm_add_norm_takes(50, [(torch.zeros(1, 1, 50), 1.0)])
+
+
 def test_the_opening_of_a_pass():
     ops = ops_of(torch.float32)
     torch.manual_seed(0)
@@ -191,6 +212,25 @@ def test_angles_of_the_latents_key_part_stay_exact_at_far_positions(rot):
     u, v, a = qr[..., 0::2], qr[..., 1::2], a[:, None, :]
     want = torch.stack([u * torch.cos(a) - v * torch.sin(a), v * torch.cos(a) + u * torch.sin(a)], -1).reshape(T, 2, rot)
     assert float((att[..., rank:rank + rot].cpu().double() - want).abs().max()) < 2e-5
+
+
+# ------------------------------------------------------------------ keys that stand out, where this design's attention looks for them
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("decoded", [False, True])
+@pytest.mark.parametrize("H,KV,hd,chunk,n,key,seen", [
+    # every head over one key/value head (a latent and a rotated part), every earlier key seen: the first of all, page borders, itself
+    (6, 1, 96, 0, 900, 0, True), (6, 1, 96, 0, 900, 15, True), (6, 1, 96, 0, 900, 16, True), (5, 1, 80, 0, 700, 699, True), (17, 1, 64, 0, 500, 3, True),
+    (3, 1, 256, 0, 600, 255, True),
+    # chunks with a sink and a gate: their first position, the one before it, the row that opens a chunk, a page's border within
+    (6, 2, 64, 104, 624, 520, True), (6, 2, 64, 104, 624, 519, False), (6, 2, 64, 104, 625, 624, True), (6, 2, 64, 104, 625, 623, False),
+    (4, 4, 48, 33, 330, 304, True), (4, 4, 48, 33, 330, 296, False), (9, 3, 128, 500, 400, 0, True)])
+def test_a_key_that_stands_out_is_seen_where_it_should_be(dtype, decoded, H, KV, hd, chunk, n, key, seen):
+    from test_livovik_gpu import _keys_case
+    rows = 1 if decoded else n
+    sinks, gate = (torch.full((H,), -9.0), torch.full((rows, H), 0.5)) if chunk else (None, None)
+    top = float(_keys_case(dtype, H, KV, hd, 16, n - rows, rows, key, chunk, sinks, gate)[:hd].min())
+    full = 25.0 if chunk else 50.0   # the key's value is 50 in every column; halved by the gate
+    assert (top > 0.8 * full) if seen else top < 0.4 * full
 
 
 # ------------------------------------------------------------------ the engine against the plain model
