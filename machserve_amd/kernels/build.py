@@ -71,14 +71,15 @@ def _hipcc() -> str:
 
 EXTRA_KINDS = {"recurrent": "recurrent.hip", "talking": "talking.hip", "latent": "latent.hip", "convattn": "convattn.hip",
                "linrec": "linrec.hip", "routed": "routed.hip", "multistream": "multistream.hip", "ssd": "ssd.hip",
-               "gated_state": "gated_state.hip"}  # libraries that only some models load
+               "gated_state": ("gated_linear.hip", "gated_delta.hip")}  # libraries that only some models load
 
 
 def _sources_of(kind: str):
     if kind == "core":
         return list(CORE_SOURCES)
     if kind in EXTRA_KINDS:
-        return ["errors.hip", EXTRA_KINDS[kind]]
+        own = EXTRA_KINDS[kind]
+        return ["errors.hip", *([own] if isinstance(own, str) else own)]
     return ["errors.hip", "attention.hip"]
 
 
