@@ -6,6 +6,16 @@ namespace ms {
 // ---- gated linear attention's decays ------------------------------------------------------------------------
 // alpha[t, c] = sigmoid(z)^(1 / tau) with z = b[c] + sum_r wt[r, c] low[t, r], low = R columns of `in` from col on; `wt` is the
 // projection transposed, [R, C].  A block takes ROWS rows and 256 channels: a weight is read once for all of its rows.
+// (the two-byte builds take the hardware's 32-bit exponential and logarithm: off by units of the last place of a decay)
+__device__ __forceinline__ float key_decay_of(float z, float inv_tau) {
+#ifdef MS_ELEM_HALF
+    const float sp = z < -20.f ? -z : __logf(1.0f + __expf(-z));
+    return __expf(-inv_tau * sp);
+#else
+    return expf(-inv_tau * softplus_f(-z));
+#endif
+}
+
 template <int ROWS>
 __global__ __launch_bounds__(256) void key_decay_kernel(Sums in, int col, const float* __restrict__ wt, const float* __restrict__ b,
                                                         float inv_tau, float* __restrict__ alpha, int T, int C, int R) {
@@ -27,7 +37,7 @@ __global__ __launch_bounds__(256) void key_decay_kernel(Sums in, int col, const 
     }
 #pragma unroll
     for (int k = 0; k < ROWS; ++k)
-        if (k < nr) alpha[(size_t)(t0 + k) * C + c] = expf(-inv_tau * softplus_f(-acc[k]));
+        if (k < nr) alpha[(size_t)(t0 + k) * C + c] = key_decay_of(acc[k], inv_tau);
 }
 
 // ---- gated linear attention over many rows ---------------------------------------------------------------------
